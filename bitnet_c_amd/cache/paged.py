@@ -238,7 +238,7 @@ class PagedCache:
 
     def commit(self, slots: Sequence[int], n_new: Sequence[int]) -> None:
         """The step has run: lengths grow; groups that keep a window give back the pages that
-        no later position can see."""
+        no later position can see (never those of the first positions that a group keeps)."""
         for s, n in zip(slots, n_new):
             self._len[s] += n
             for g in self.groups:
@@ -246,7 +246,7 @@ class PagedCache:
                     first_visible = self._len[s] - g.need.window + 1     # for the next position
                     pl = g.pages[s]
                     for i in range(len(pl)):
-                        if pl[i] >= 0 and PAGE * i + PAGE - 1 < first_visible:
+                        if pl[i] >= 0 and PAGE * i >= g.need.keep_first and PAGE * i + PAGE - 1 < first_visible:
                             g.pool.give_back([pl[i]])
                             pl[i] = -1
                             self._touch(s)

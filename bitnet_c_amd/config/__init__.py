@@ -1,4 +1,4 @@
-"""Typed configurations and the architecture registry; importing registers "llama", "Sunusun", "Sonodra", "Fazopel" and "Mutirax"."""
+"""Typed configurations and the architecture registry; importing registers "llama", "Sunusun", "Sonodra", "Fazopel", "Mutirax" and "Pafutar"."""
 from .base import (Architecture, ConfigError, architecture_for, architecture_names, load_config,
                    read_config_json, register_architecture)
 from .llama import LlamaConfig, RopeScaling
@@ -6,4 +6,5 @@ from .sunusun import SunusunConfig
 from .sonodra import SonodraConfig
 from .fazopel import FazopelConfig
 from .mutirax import MutiraxConfig
+from .pafutar import PafutarConfig
 from . import llama_plan  # noqa: F401  (registration)

@@ -6,20 +6,23 @@
 //
 // A wave owns one tile of up to 16 query tokens of one head and walks the keys 0 .. last query in blocks of 32 (with a
 // window w > 0 a query at position i sees the keys i - w + 1 .. i only, and the walk begins at the block of the tile's
-// first visible key):
+// first visible key; with keep_first k > 0 the keys 0 .. k - 1 stay in sight, and the walk begins at block 0 and leaps from
+// the block behind the kept keys to the window's first):
 //   S^T = K . Q^T      two tiles of 16 keys x 16 queries; tile h holds the block's keys 8 (i / 4) + 4 h + i % 4 in its
 //                      row i, so that lane group g ends up with the scores of keys 8 g .. 8 g + 7 of its query column:
 //                      what the second product wants from it as its operand, without any exchange
-//   s = S scale - a[h] ln(1 + b[h] (i - j)), masked above the diagonal; online softmax in base 2, float32
+//   s = S scale - a[h] ln(1 + b[h] (i - j)) or S scale - a[h] (i - j), masked above the diagonal; online softmax in base 2, float32
 //   O^T += V^T . P^T   vd / 16 tiles; the weights' sums from the matrix cores as well (a tile of ones times P^T), so that
 //                      numerator and denominator see the same bf16 weights
-// and at the end the sink (one more term of score 0 without a value) joins the sums, then O / l is stored.
+// and at the end the sink (one more term of score 0 without a value) joins the sums, then O / l is stored, times
+// sigmoid(gate) element by element when the mixer gates its heads' outputs.
 //
 // Decode form (attn_general_decode_kernel): the 16 columns of a tile are the query heads that share a kv head (the one new
 // token of a sequence), so a block of keys and values is loaded once for all of them: a wave owns (sequence, kv head,
 // sixteen of its heads, split of the keys) and either stores the result or, with the keys split over gridDim.z, leaves
 // unnormalised sums with their maximum and weight sum for attn_general_combine_kernel, which merges the splits in index
-// order.  Splits are runs of whole pages; with a window they are counted from the page of the window's first key.
+// order.  Splits are runs of whole pages; with a window they are counted from the page of the window's first key, and the
+// kept first keys are the first split's.
 // Every other shape or type is the vector kernel's (attn_rows.hip).
 #include "common.h"
 #include <math.h>
@@ -39,16 +42,39 @@ struct GenArgs {
     const int* block_table;   // [seqs, bt_stride]
     const int* tiles;         // [n, 4]: sequence, first row, rows <= 16, position of the first
     const float* dist_a;      // [H] or null
-    const float* dist_b;
+    const float* dist_b;      // [H], or null: the bias is linear, dist_a[h] (i - j)
+    const bf16* gate;         // [T, gate_stride] beside out's columns, or null: out times sigmoid(gate)
+    int gate_stride;
     int q_stride, out_stride, bt_stride, H, Hkv;
     float scale;
     int sink;                 // 1: one more term without a value in the softmax's denominator, exp(sink_values[head])
     const float* sink_values; // [H] float32, or null: the term's score is 0
     int window;               // 0: every earlier key; else the last `window` positions, the query's own included
+    int keep_first;           // with a window: the first keep_first positions stay visible however far back they are
 };
 
 __device__ __forceinline__ bf16x8 ag_ld16(const bf16* p) {
     return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p));
+}
+
+// the score's distance bias in the exponent's base 2; a ln(x) log2(e) = a log2(x)
+__device__ __forceinline__ float ag_bias2(float a, float b, bool linear, float dist) {
+    return linear ? a * AG_LOG2E * dist : a * __log2f(1.0f + b * dist);
+}
+
+// four consecutive outputs of a head and, with a gate, times the sigmoids of the four gate values beside them:
+// one 8-byte store
+__device__ __forceinline__ void ag_store4(bf16* op, const bf16* gp, float x0, float x1, float x2, float x3) {
+    if (gp) {
+        const uint2 gw = *reinterpret_cast<const uint2*>(gp);
+        x0 /= 1.0f + __expf(-bf16lo_to_f32(gw.x)); x1 /= 1.0f + __expf(-bf16hi_to_f32(gw.x));
+        x2 /= 1.0f + __expf(-bf16lo_to_f32(gw.y)); x3 /= 1.0f + __expf(-bf16hi_to_f32(gw.y));
+    }
+    const bf16 o0 = __float2bfloat16(x0), o1 = __float2bfloat16(x1), o2 = __float2bfloat16(x2), o3 = __float2bfloat16(x3);
+    uint2 w;
+    w.x = (uint32_t)__builtin_bit_cast(unsigned short, o0) | ((uint32_t)__builtin_bit_cast(unsigned short, o1) << 16);
+    w.y = (uint32_t)__builtin_bit_cast(unsigned short, o2) | ((uint32_t)__builtin_bit_cast(unsigned short, o3) << 16);
+    *reinterpret_cast<uint2*>(op) = w;
 }
 
 template <int DC, int DT>     // hs = 32 DC, vd = 16 DT
@@ -72,7 +98,8 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
         for (int c = 0; c < DC; ++c) qf[c] = ag_ld16(qp + 32 * c);
     }
     const float scale2 = a.scale * AG_LOG2E;
-    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a ? a.dist_b[head] : 0.f;
+    const bool linear = a.dist_b == nullptr;
+    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a && !linear ? a.dist_b[head] : 0.f;
     f32x4 acc[DT];
 #pragma unroll
     for (int t = 0; t < DT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -92,16 +119,18 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
     };
     const int k_lo = a.window > 0 ? max(0, pos0 - a.window + 1) & ~31 : 0;      // the block of the first key any row sees
     const int q_lo = a.window > 0 ? qpos - a.window : -1;                        // keys at or below this are out of sight
-    ask_keys(k_lo);
+    const int keep = a.window > 0 ? min(a.keep_first, k_hi) : 0;                 // keys below this stay in sight
+    auto leap = [&](int kb) { return kb >= keep && kb < k_lo ? k_lo : kb; };     // past what no row of the tile sees
     const int last_block = ((k_hi - 1) / 32) * 32;
-    for (int kb = k_lo; kb < k_hi; kb += 32) {
+    ask_keys(leap(0));
+    for (int kb = leap(0); kb < k_hi; kb = leap(kb + 32)) {
         const int page = a.block_table[(size_t)seq * a.bt_stride + kb / BN_PAGE];
         const int off = kb % BN_PAGE;
         const bf16* vbase = a.v_pages + (((size_t)page * a.Hkv + kvh) * VD + i) * BN_PAGE + off + 8 * g;
         bf16x8 k0[DC], k1[DC];
 #pragma unroll
         for (int c = 0; c < DC; ++c) { k0[c] = kn0[c]; k1[c] = kn1[c]; }
-        ask_keys(min(kb + 32, last_block));
+        ask_keys(min(leap(kb + 32), last_block));
         f32x4 st0 = (f32x4){0.f, 0.f, 0.f, 0.f}, st1 = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int c = 0; c < DC; ++c) {
@@ -119,8 +148,8 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
         for (int e = 0; e < 8; ++e) {
             const int key = kb + 8 * g + e;
             float v = (e < 4 ? st0[e & 3] : st1[e & 3]) * scale2;
-            if (a.dist_a) v -= ba * __log2f(1.0f + bb * (float)(qpos - key));     // a ln(x) log2(e) = a log2(x)
-            if (!col_ok || key > qpos || key >= k_hi || key <= q_lo) v = -INFINITY;
+            if (a.dist_a) v -= ag_bias2(ba, bb, linear, (float)(qpos - key));
+            if (!col_ok || key > qpos || key >= k_hi || (key <= q_lo && key >= keep)) v = -INFINITY;
             s[e] = v;
             mx = fmaxf(mx, v);
         }
@@ -176,15 +205,10 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
     if (!col_ok) return;
     // acc[t][r] = O^T[value column 16 t + 4 g + r][query i]: four consecutive columns, one 8-byte store
     bf16* op = a.out + (size_t)(row0 + i) * a.out_stride + (size_t)head * VD + 4 * g;
+    const bf16* gp = a.gate ? a.gate + (size_t)(row0 + i) * a.gate_stride + (size_t)head * VD + 4 * g : nullptr;
 #pragma unroll
-    for (int t = 0; t < DT; ++t) {
-        const bf16 o0 = __float2bfloat16(acc[t][0] * inv), o1 = __float2bfloat16(acc[t][1] * inv);
-        const bf16 o2 = __float2bfloat16(acc[t][2] * inv), o3 = __float2bfloat16(acc[t][3] * inv);
-        uint2 w;
-        w.x = (uint32_t)__builtin_bit_cast(unsigned short, o0) | ((uint32_t)__builtin_bit_cast(unsigned short, o1) << 16);
-        w.y = (uint32_t)__builtin_bit_cast(unsigned short, o2) | ((uint32_t)__builtin_bit_cast(unsigned short, o3) << 16);
-        *reinterpret_cast<uint2*>(op + 16 * t) = w;
-    }
+    for (int t = 0; t < DT; ++t)
+        ag_store4(op + 16 * t, gp ? gp + 16 * t : nullptr, acc[t][0] * inv, acc[t][1] * inv, acc[t][2] * inv, acc[t][3] * inv);
 }
 
 struct GenDecodeArgs {
@@ -195,11 +219,13 @@ struct GenDecodeArgs {
     const int* block_table;   // [n_seqs, bt_stride]
     const int* seq_lens;      // [n_seqs] keys in the cache, the new one included; 0: a padding row
     const float* dist_a;
-    const float* dist_b;
+    const float* dist_b;      // null: the bias is linear
+    const bf16* gate;         // [n_seqs, gate_stride] or null
+    int gate_stride;
     float* part_o;            // [n_seqs H, n_splits, vd]   (n_splits > 1)
     float* part_ml;           // [n_seqs H, n_splits, 2]: maximum (natural exponent) and sum of the weights
     const int* max_len;       // != null: the longest sequence's key count; the keys per split follow from it
-    int q_stride, out_stride, bt_stride, H, Hkv, n_splits, chunk, window, sink;
+    int q_stride, out_stride, bt_stride, H, Hkv, n_splits, chunk, window, keep_first, sink;
     const float* sink_values; // [H] float32, or null (score 0)
     float scale;
 };
@@ -214,9 +240,10 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
     const bool col_ok = 16 * ht + i < G;                 // this lane's column is a head that exists
     const int head = kvh * G + min(16 * ht + i, G - 1);
     const int len = a.seq_lens[seq], qpos = len - 1;
-    int k_lo = 0, k_hi = 0;
+    int k_lo = 0, k_hi = 0, keep = 0;                    // this wave's keys: k_lo .. k_hi - 1, and 0 .. keep - 1
     if (len > 0) {
         const int lo = a.window > 0 ? max(0, len - a.window) : 0;
+        if (split == 0 && a.window > 0) keep = min(a.keep_first, lo);
         if (a.n_splits > 1) {
             const int chunk = a.max_len ? bn_split_chunk(*a.max_len, a.n_splits) : a.chunk;
             const int base = a.window > 0 ? (lo / BN_PAGE) * BN_PAGE : 0;
@@ -248,7 +275,8 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
         for (int c = 0; c < DC; ++c) qf[c] = ag_ld16(qp + 32 * c);
     }
     const float scale2 = a.scale * AG_LOG2E;
-    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a ? a.dist_b[head] : 0.f;
+    const bool linear = a.dist_b == nullptr;
+    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a && !linear ? a.dist_b[head] : 0.f;
     f32x4 acc[DT];
 #pragma unroll
     for (int t = 0; t < DT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -263,14 +291,15 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
         for (int c = 0; c < DC; ++c) { kn0[c] = ag_ld16(kbase + 32 * c); kn1[c] = ag_ld16(kbase + 4 * HS + 32 * c); }
     };
     const int first_block = k_lo & ~31, last_block = ((k_hi - 1) / 32) * 32;
-    ask_keys(first_block);
-    for (int kb = first_block; kb < k_hi; kb += 32) {
+    auto leap = [&](int kb) { return kb >= keep && kb < first_block ? first_block : kb; };
+    ask_keys(leap(0));
+    for (int kb = leap(0); kb < k_hi; kb = leap(kb + 32)) {
         const int page = a.block_table[(size_t)seq * a.bt_stride + kb / BN_PAGE];
         const bf16* vbase = a.v_pages + (((size_t)page * a.Hkv + kvh) * VD + i) * BN_PAGE + kb % BN_PAGE + 8 * g;
         bf16x8 k0[DC], k1[DC];
 #pragma unroll
         for (int c = 0; c < DC; ++c) { k0[c] = kn0[c]; k1[c] = kn1[c]; }
-        ask_keys(min(kb + 32, last_block));
+        ask_keys(min(leap(kb + 32), last_block));
         f32x4 st0 = (f32x4){0.f, 0.f, 0.f, 0.f}, st1 = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int c = 0; c < DC; ++c) {
@@ -286,8 +315,8 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
         for (int e = 0; e < 8; ++e) {
             const int key = kb + 8 * g + e;
             float v = (e < 4 ? st0[e & 3] : st1[e & 3]) * scale2;
-            if (a.dist_a) v -= ba * __log2f(1.0f + bb * (float)(qpos - key));
-            if (!col_ok || key < k_lo || key >= k_hi) v = -INFINITY;
+            if (a.dist_a) v -= ag_bias2(ba, bb, linear, (float)(qpos - key));
+            if (!col_ok || (key < k_lo && key >= keep) || key >= k_hi) v = -INFINITY;
             s[e] = v;
             mx = fmaxf(mx, v);
         }
@@ -348,24 +377,20 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
     }
     const float inv = l > 0.f ? fa / l : 0.f;
     bf16* op = a.out + (size_t)seq * a.out_stride + (size_t)head * VD + 4 * g;
+    const bf16* gp = a.gate ? a.gate + (size_t)seq * a.gate_stride + (size_t)head * VD + 4 * g : nullptr;
 #pragma unroll
-    for (int t = 0; t < DT; ++t) {
-        const bf16 o0 = __float2bfloat16(acc[t][0] * inv), o1 = __float2bfloat16(acc[t][1] * inv);
-        const bf16 o2 = __float2bfloat16(acc[t][2] * inv), o3 = __float2bfloat16(acc[t][3] * inv);
-        uint2 w;
-        w.x = (uint32_t)__builtin_bit_cast(unsigned short, o0) | ((uint32_t)__builtin_bit_cast(unsigned short, o1) << 16);
-        w.y = (uint32_t)__builtin_bit_cast(unsigned short, o2) | ((uint32_t)__builtin_bit_cast(unsigned short, o3) << 16);
-        *reinterpret_cast<uint2*>(op + 16 * t) = w;
-    }
+    for (int t = 0; t < DT; ++t)
+        ag_store4(op + 16 * t, gp ? gp + 16 * t : nullptr, acc[t][0] * inv, acc[t][1] * inv, acc[t][2] * inv, acc[t][3] * inv);
 }
 
-// out[row, d] = sum_s e^(m_s - m) o_s[d] / (sum_s e^(m_s - m) l_s [+ e^(-m) for the sink]), the splits in index order;
+// out[row, d] = sum_s e^(m_s - m) o_s[d] / (sum_s e^(m_s - m) l_s [+ e^(-m) for the sink]) [sigmoid(gate)], the splits in index order;
 // one wave a (token, head) row, a lane four value columns at a time
 __global__ __launch_bounds__(BN_WAVE) void attn_general_combine_kernel(bf16* __restrict__ out, int out_stride,
                                                                        const float* __restrict__ part_o,
                                                                        const float* __restrict__ part_ml, int H, int vd,
                                                                        int n_splits, int sink,
-                                                                       const float* __restrict__ sink_values) {
+                                                                       const float* __restrict__ sink_values,
+                                                                       const bf16* __restrict__ gate, int gate_stride) {
     const int row = blockIdx.x, tok = row / H, head = row - tok * H;
     const float* ml = part_ml + (size_t)row * n_splits * 2;
     const float sv = sink && sink_values ? sink_values[head] : 0.f;
@@ -386,8 +411,8 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_combine_kernel(bf16* __r
             }
         }
         bf16* op = out + (size_t)tok * out_stride + (size_t)head * vd + d;
-        op[0] = __float2bfloat16(num.x * inv); op[1] = __float2bfloat16(num.y * inv);
-        op[2] = __float2bfloat16(num.z * inv); op[3] = __float2bfloat16(num.w * inv);
+        ag_store4(op, gate ? gate + (size_t)tok * gate_stride + (size_t)head * vd + d : nullptr, num.x * inv, num.y * inv, num.z * inv,
+                  num.w * inv);
     }
 }
 
@@ -414,12 +439,15 @@ static int ag_launch_dt(const GenArgs& a, int vd, dim3 grid, hipStream_t s) {
 extern "C" int bn_attn_general_prompt(const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
                                       const void* v_pages, const int* block_table, int bt_stride, const int* tiles, int n_tiles,
                                       int H, int Hkv, int hs, int vd, float scale, const float* dist_a, const float* dist_b,
-                                      int sink, const float* sink_values, int window, hipStream_t s) {
-    if (n_tiles <= 0 || H <= 0 || Hkv <= 0 || H % Hkv || window < 0 || !bn_attn_general_supports(hs, vd)) return BN_ERR_ARG;
-    if (!q || !out || !k_pages || !v_pages || !block_table || !tiles || (dist_a == nullptr) != (dist_b == nullptr)) return BN_ERR_ARG;
+                                      int sink, const float* sink_values, int window, int keep_first, const void* gate,
+                                      int gate_stride, hipStream_t s) {
+    if (n_tiles <= 0 || H <= 0 || Hkv <= 0 || H % Hkv || window < 0 || keep_first < 0 || !bn_attn_general_supports(hs, vd)) return BN_ERR_ARG;
+    if (!q || !out || !k_pages || !v_pages || !block_table || !tiles || (dist_b && !dist_a)) return BN_ERR_ARG;
     if (q_stride % 8 || out_stride % 4 || (((uintptr_t)q | (uintptr_t)k_pages | (uintptr_t)v_pages) & 15) || ((uintptr_t)out & 7))
         return BN_ERR_ARG;
+    if (gate && (gate_stride % 4 || ((uintptr_t)gate & 7))) return BN_ERR_ARG;
     GenArgs a;
+    a.gate = (const bf16*)gate; a.gate_stride = gate_stride; a.keep_first = keep_first;
     a.q = (const bf16*)q; a.out = (bf16*)out; a.k_pages = (const bf16*)k_pages; a.v_pages = (const bf16*)v_pages;
     a.block_table = block_table; a.tiles = tiles; a.dist_a = dist_a; a.dist_b = dist_b;
     a.q_stride = q_stride; a.out_stride = out_stride; a.bt_stride = bt_stride; a.H = H; a.Hkv = Hkv;
@@ -456,16 +484,18 @@ static int ag_launch_decode_dt(const GenDecodeArgs& a, int vd, dim3 grid, hipStr
 extern "C" int bn_attn_general_decode(const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
                                       const void* v_pages, const int* block_table, int bt_stride, const int* seq_lens, int n_seqs,
                                       int H, int Hkv, int hs, int vd, float scale, const float* dist_a, const float* dist_b,
-                                      int sink, const float* sink_values, int window, int n_splits, int chunk, float* part_o, float* part_ml,
-                                      const int* max_len, hipStream_t s) {
-    if (n_seqs <= 0 || H <= 0 || Hkv <= 0 || H % Hkv || window < 0 || n_splits < 1 || !bn_attn_general_supports(hs, vd)) return BN_ERR_ARG;
-    if (!q || !out || !k_pages || !v_pages || !block_table || !seq_lens || (dist_a == nullptr) != (dist_b == nullptr)) return BN_ERR_ARG;
+                                      int sink, const float* sink_values, int window, int keep_first, const void* gate, int gate_stride,
+                                      int n_splits, int chunk, float* part_o, float* part_ml, const int* max_len, hipStream_t s) {
+    if (n_seqs <= 0 || H <= 0 || Hkv <= 0 || H % Hkv || window < 0 || keep_first < 0 || n_splits < 1 || !bn_attn_general_supports(hs, vd)) return BN_ERR_ARG;
+    if (!q || !out || !k_pages || !v_pages || !block_table || !seq_lens || (dist_b && !dist_a)) return BN_ERR_ARG;
     if (q_stride % 8 || out_stride % 4 || (((uintptr_t)q | (uintptr_t)k_pages | (uintptr_t)v_pages) & 15) || ((uintptr_t)out & 7))
         return BN_ERR_ARG;
     if (n_splits > 1 && (!part_o || !part_ml || ((uintptr_t)part_o & 15) || (!max_len && (chunk <= 0 || chunk % BN_PAGE)))) return BN_ERR_ARG;
     const int head_tiles = (H / Hkv + 15) / 16;
     if ((long long)Hkv * head_tiles > 65535 || n_splits > 65535) return BN_ERR_ARG;
+    if (gate && (gate_stride % 4 || ((uintptr_t)gate & 7))) return BN_ERR_ARG;
     GenDecodeArgs a;
+    a.gate = (const bf16*)gate; a.gate_stride = gate_stride; a.keep_first = keep_first;
     a.q = (const bf16*)q; a.out = (bf16*)out; a.k_pages = (const bf16*)k_pages; a.v_pages = (const bf16*)v_pages;
     a.block_table = block_table; a.seq_lens = seq_lens; a.dist_a = dist_a; a.dist_b = dist_b; a.part_o = part_o; a.part_ml = part_ml;
     a.max_len = n_splits > 1 ? max_len : nullptr;
@@ -482,6 +512,6 @@ extern "C" int bn_attn_general_decode(const void* q, int q_stride, void* out, in
     }
     if (rc != 0 || n_splits == 1) return rc;
     hipLaunchKernelGGL(attn_general_combine_kernel, dim3(n_seqs * H), dim3(BN_WAVE), 0, s, (bf16*)out, out_stride, part_o, part_ml,
-                       H, vd, n_splits, sink ? 1 : 0, sink ? sink_values : nullptr);
+                       H, vd, n_splits, sink ? 1 : 0, sink ? sink_values : nullptr, (const bf16*)gate, gate_stride);
     return bn_launch_status();
 }

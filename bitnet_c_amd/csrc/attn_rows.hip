@@ -34,6 +34,7 @@ struct AttnArgs {
     int GT;                   // heads of one kv group handled together (power of two <= RT)
     int KT;                   // keys per tile: 16, 32 or 64
     int window;               // 0 = all earlier keys, else the last `window` of them
+    int keep_first;           // with a window: the first keep_first positions stay visible however far back they are
     int n_splits, chunk;      // keys per split, a multiple of BN_PAGE
     int v_transposed;         // V pages are [page, kv_head, hs, BN_PAGE]
     float scale;
@@ -44,7 +45,7 @@ struct AttnArgs {
     int vd;                   // width of a value head (the keys' hs unless the mixer says otherwise); out, part_o and the
                               // value pages are vd wide
     const float* dist_a;      // [H] or null: a bias that grows with the distance is taken off the score of query i and
-    const float* dist_b;      // key j: dist_a[h] * ln(1 + dist_b[h] * (i - j))
+    const float* dist_b;      // key j: dist_a[h] * ln(1 + dist_b[h] * (i - j)); dist_b null: dist_a[h] * (i - j)
     int sink;                 // 1: the softmax has one more term without a value: exp(sink_values[head]) joins its denominator
     const float* sink_values; // [H] float32, or null: the term's score is 0 for every head
 };
@@ -144,7 +145,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_rows_kernel(AttnArgs a) {
         for (int idx = tid; idx < KT * (kstride + vstride); idx += ATT_THREADS) k_s[idx] = from_f32<T>(0.f);
 
     // keys this workgroup visits
-    int lo = 0, hi = 0;
+    int lo = 0, hi = 0, keep = 0;                        // keys lo .. hi - 1, and the kept ones 0 .. keep - 1
     if (pos0 >= 0 && n_tok > 0) {
         hi = pos0 + n_tok;                                        // exclusive
         lo = a.window > 0 ? max(0, pos0 + 1 - a.window) : 0;      // first key of the first row
@@ -154,6 +155,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_rows_kernel(AttnArgs a) {
         const int base = (a.window > 0 && a.n_splits > 1 && !a.tiles) ? (lo / BN_PAGE) * BN_PAGE : 0;
         lo = max(lo, base + split * chunk);
         hi = min(hi, base + (split + 1) * chunk);
+        if (a.window > 0 && split == 0) keep = min(a.keep_first, hi);      // the kept keys are the first split's
     }
 
     // phase C ownership: thread -> (jp, dp): keys jp, jp+JP, ...; output dims 2dp, 2dp+1
@@ -221,7 +223,10 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_rows_kernel(AttnArgs a) {
     const int lane = tid & 63, wave = tid >> 6;
     __syncthreads();
 
-    for (int j0 = (lo / KT) * KT; j0 < hi; j0 += KT) {
+    // the walk goes from tile to tile of keys; behind the kept keys it leaps to the tile of the first other visible one
+    const int lo_tile = (lo / KT) * KT;
+    auto leap = [&](int j) { return j >= keep && j < lo_tile ? lo_tile : j; };
+    for (int j0 = leap(0); j0 < hi; j0 = leap(j0 + KT)) {
         // ---- load the K and V tile (rows j0 .. j0+KT-1 of one page) ----
         {
             const int page = a.block_table[(size_t)seq * a.bt_stride + j0 / BN_PAGE];
@@ -305,12 +310,13 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_rows_kernel(AttnArgs a) {
                 if ((r % P) == pa) {
                     const int i = r / GT, g = r - i * GT;
                     const int qpos = pos0 + i;
-                    bool ok = (i < n_tok) && (ht * GT + g < G) && key <= qpos && key >= lo && key < hi;
-                    if (a.window > 0) ok = ok && (key > qpos - a.window);
+                    bool ok = (i < n_tok) && (ht * GT + g < G) && key <= qpos && key < hi;
+                    ok = ok && (key < keep || (key >= lo && (a.window <= 0 || key > qpos - a.window)));
                     float sc = dot[r] * a.scale;
                     if (a.dist_a && ok) {
                         const int head = kvh * G + ht * GT + g;
-                        sc -= a.dist_a[head] * logf(1.0f + a.dist_b[head] * (float)(qpos - key));
+                        const float dist = (float)(qpos - key);
+                        sc -= a.dist_a[head] * (a.dist_b ? logf(1.0f + a.dist_b[head] * dist) : dist);
                     }
                     s_s[r * KT + ja] = ok ? sc : -INFINITY;
                 }
@@ -363,8 +369,9 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_rows_kernel(AttnArgs a) {
         }
         __syncthreads();
         // a run of keys ends here and more keys follow (one workgroup walks several runs: a prompt step, or a decode step
-        // whose keys are not split): fold it
-        if (a.fold > 0 && a.n_splits == 1 && (j0 + KT) % a.fold == 0 && j0 + KT < hi) fold_run();
+        // whose keys are not split): fold it.  A leap may end a run before its last tile.
+        const int next = leap(j0 + KT);
+        if (a.fold > 0 && a.n_splits == 1 && next < hi && next / a.fold != j0 / a.fold) fold_run();
     }
 
     const bool folded = a.fold > 0 && a.n_splits == 1;
@@ -508,15 +515,15 @@ extern "C" int bn_attn_rows(int dtype, const void* q, int q_stride, void* out, i
                             int n_tokens, int H, int Hkv, int hs, int RT, int GT, int window,
                             float scale, int n_splits, int chunk, float* part_o, float* part_ml,
                             int v_transposed, const int* max_len, int fold, int vd, const float* dist_a,
-                            const float* dist_b, int sink, const float* sink_values, hipStream_t s) {
+                            const float* dist_b, int sink, const float* sink_values, int keep_first, hipStream_t s) {
     if (vd == 0) vd = hs;
-    if (vd < 2 || vd > BN_MAX_HEAD_DIM || vd % 2 || (dist_a == nullptr) != (dist_b == nullptr)) return BN_ERR_ARG;
+    if (vd < 2 || vd > BN_MAX_HEAD_DIM || vd % 2 || (dist_b && !dist_a)) return BN_ERR_ARG;
     if (n_tiles <= 0 || n_tokens <= 0 || H <= 0 || Hkv <= 0 || H % Hkv) return BN_ERR_ARG;
     // fold mode: runs of whole pages; a split is one run, and the runs' length does not follow the longest sequence
     if (fold < 0 || fold % BN_PAGE || (fold > 0 && n_splits > 1 && (chunk != fold || max_len))) return BN_ERR_ARG;
     if (hs < 2 || hs > BN_MAX_HEAD_DIM || hs % 2) return BN_ERR_ARG;
     if (GT <= 0 || GT > RT || (GT & (GT - 1)) || RT > 16 || (RT & (RT - 1))) return BN_ERR_ARG;
-    if (n_splits < 1 || window < 0) return BN_ERR_ARG;
+    if (n_splits < 1 || window < 0 || keep_first < 0) return BN_ERR_ARG;
     if (n_splits > 1 && (!part_o || !part_ml || (!max_len && (chunk <= 0 || chunk % BN_PAGE)))) return BN_ERR_ARG;
     if (!tiles && !seq_lens) return BN_ERR_ARG;
     if (max_len && tiles) return BN_ERR_ARG;
@@ -526,7 +533,7 @@ extern "C" int bn_attn_rows(int dtype, const void* q, int q_stride, void* out, i
     a.block_table = block_table; a.seq_lens = seq_lens; a.tiles = tiles;
     a.part_o = part_o; a.part_ml = part_ml;
     a.q_stride = q_stride; a.out_stride = out_stride; a.bt_stride = bt_stride;
-    a.H = H; a.Hkv = Hkv; a.hs = hs; a.GT = GT; a.window = window;
+    a.H = H; a.Hkv = Hkv; a.hs = hs; a.GT = GT; a.window = window; a.keep_first = keep_first;
     a.n_splits = n_splits; a.chunk = n_splits > 1 ? chunk : 0x40000000;
     a.scale = scale;
     a.v_transposed = v_transposed;

@@ -534,6 +534,40 @@ extern "C" int bn_embed_gather_sinusoid(int dtype, void* x, const void* table, c
     return bn_launch_status();
 }
 
+// ---- an embedding with a learned position vector -----------------------------------------------------------------
+// x[t, e] = table[token, e] * scale + pos_table[position, e] (the position's row is not scaled).  A row without a position
+// (< 0: padding), or with one that the table does not have, gets none; the step function admits no such position.
+template <typename T>
+__global__ void embed_gather_learned_kernel(float* __restrict__ x, const T* __restrict__ table,
+                                            const int* __restrict__ tokens, const int* __restrict__ positions,
+                                            const T* __restrict__ pos_table, int dim, int vocab, int n_pos, float scale) {
+    const int t = blockIdx.x;
+    const int tok = tokens[t], pos = positions[t];
+    float* row = x + (size_t)t * dim;
+    const bool known = tok >= 0 && tok < vocab, placed = pos >= 0 && pos < n_pos;
+    const T* src = table + (size_t)(known ? tok : 0) * dim;
+    const T* prow = pos_table + (size_t)(placed ? pos : 0) * dim;
+    for (int e = threadIdx.x; e < dim; e += blockDim.x) {
+        const float a = to_f32(src[e]), b = to_f32(prow[e]);
+        row[e] = fmaf(known ? a : 0.f, scale, placed ? b : 0.f);
+    }
+}
+
+extern "C" int bn_embed_gather_learned(int dtype, void* x, const void* table, const int* tokens, const int* positions,
+                                       const void* pos_table, int n_tokens, int dim, int vocab, int n_pos, float scale,
+                                       hipStream_t s) {
+    if (n_tokens <= 0 || dim <= 0 || vocab <= 0 || n_pos <= 0 || !x || !table || !tokens || !positions || !pos_table) return BN_ERR_ARG;
+    if (dtype == BN_DT_F32)
+        hipLaunchKernelGGL(embed_gather_learned_kernel<float>, dim3(n_tokens), dim3(256), 0, s, (float*)x, (const float*)table,
+                           tokens, positions, (const float*)pos_table, dim, vocab, n_pos, scale);
+    else if (dtype == BN_DT_BF16)
+        hipLaunchKernelGGL(embed_gather_learned_kernel<bf16>, dim3(n_tokens), dim3(256), 0, s, (float*)x, (const bf16*)table,
+                           tokens, positions, (const bf16*)pos_table, dim, vocab, n_pos, scale);
+    else
+        return BN_ERR_DTYPE;
+    return bn_launch_status();
+}
+
 // ---- activations of one argument (bn_unary_act of common.h) over a tensor ----------------------------------------
 template <typename T>
 __global__ void unary_act_kernel(T* __restrict__ out, const T* __restrict__ in, size_t n, int kind) {

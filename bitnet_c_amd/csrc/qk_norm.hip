@@ -10,8 +10,11 @@
 //   k_g <- rot_p(k_g / rms * wk)                       -> page of position p
 //   v_g                                                 -> page of position p
 //
+// bias: one float32 number per query and key column, added to the projections before anything else happens to them (so
+// values that are the keys have it too).  head_temp: one number per query head that multiplies the finished query.
+//
 // v_from_k: the values are the key projections themselves, as projected (before the key's norm and rotation): qkv then
-// holds no value heads, and kv head g's value is read from its key's columns, which this kernel leaves as they arrived.
+// holds no value heads, and kv head g's value is its key's columns (plus their bias), which this kernel leaves as they arrived.
 //
 // Pages hold a row per position for the keys, [page, kv head, BN_PAGE, hs]; the values lie the same way ("rows" layout,
 // [page, kv head, BN_PAGE, vd]) or transposed ([page, kv head, vd, BN_PAGE]), as the caller says.
@@ -32,6 +35,8 @@ struct QkNormArgs {
     const float* wq;          // [hs], or [H hs] when norm_all; null: no norm
     const float* wk;          // [hs], or [Hkv hs]
     const float* inv_freq;    // [rope_dims / 2]; null: no rotation
+    const float* bias;        // [(H + Hkv) hs] or null
+    const float* head_temp;   // [H] or null
     int ld, bt_stride, H, Hkv, hs, vd;
     int v_transposed;         // the values' pages are [page, kv head, vd, BN_PAGE]
     int norm_all;             // the norms run over the whole projection instead of over each head
@@ -66,8 +71,14 @@ __global__ __launch_bounds__(QKN_MAX_WAVES * BN_WAVE) void qk_norm_store_kernel(
     if (a.norm_all && a.wq) {
         const int nq = a.H * a.hs, nk = a.Hkv * a.hs;
         float sq = 0.f, sk = 0.f;
-        for (int d = threadIdx.x; d < nq; d += blockDim.x) { const float x = to_f32(row[d]); sq = fmaf(x, x, sq); }
-        for (int d = threadIdx.x; d < nk; d += blockDim.x) { const float x = to_f32(row[nq + d]); sk = fmaf(x, x, sk); }
+        for (int d = threadIdx.x; d < nq; d += blockDim.x) {
+            const float x = to_f32(row[d]) + (a.bias ? a.bias[d] : 0.f);
+            sq = fmaf(x, x, sq);
+        }
+        for (int d = threadIdx.x; d < nk; d += blockDim.x) {
+            const float x = to_f32(row[nq + d]) + (a.bias ? a.bias[nq + d] : 0.f);
+            sk = fmaf(x, x, sk);
+        }
         sq = block_sum(sq, scratch);
         sk = block_sum(sk, scratch);
         fq = 1.0f / sqrtf(sq / (float)nq + a.eps);
@@ -82,17 +93,19 @@ __global__ __launch_bounds__(QKN_MAX_WAVES * BN_WAVE) void qk_norm_store_kernel(
         if (is_q || is_k) {
             if (is_k && !a.k_pages) continue;
             T* v = row + (size_t)head * a.hs;
+            const float* bias = a.bias ? a.bias + (size_t)head * a.hs : nullptr;
             const float* w = is_q ? a.wq : a.wk;
             if (w && a.norm_all) w += (size_t)(is_q ? head : head - a.H) * a.hs;
             float f = is_q ? fq : fk;
             if (w && !a.norm_all) {
                 float ss = 0.f;
-                for (int d = lane; d < a.hs; d += BN_WAVE) { const float x = to_f32(v[d]); ss = fmaf(x, x, ss); }
+                for (int d = lane; d < a.hs; d += BN_WAVE) { const float x = to_f32(v[d]) + (bias ? bias[d] : 0.f); ss = fmaf(x, x, ss); }
                 ss = wave_sum(ss);
                 f = 1.0f / sqrtf(ss / (float)a.hs + a.eps);
             }
             float temp = 1.0f;
             if (is_q && a.temp_every > 0) temp = 1.0f + a.temp_coef * logf((float)((pos + 1) / a.temp_every) + 1.0f);
+            if (is_q && a.head_temp) temp *= a.head_temp[head];
             // the whole head first (a rotation reads its partner, which another lane or a later turn overwrites)
             float xs[QKN_PER_LANE], ps[QKN_PER_LANE];
 #pragma unroll
@@ -100,11 +113,11 @@ __global__ __launch_bounds__(QKN_MAX_WAVES * BN_WAVE) void qk_norm_store_kernel(
                 const int d = lane + BN_WAVE * j;
                 xs[j] = ps[j] = 0.f;
                 if (d < a.hs) {
-                    xs[j] = to_f32(v[d]);
+                    xs[j] = to_f32(v[d]) + (bias ? bias[d] : 0.f);
                     if (w) xs[j] = xs[j] * f * w[d];
                     if (d < rd) {
                         const int pd = a.rope_interleaved ? (d ^ 1) : (d < half ? d + half : d - half);
-                        ps[j] = to_f32(v[pd]);
+                        ps[j] = to_f32(v[pd]) + (bias ? bias[pd] : 0.f);
                         if (w) ps[j] = ps[j] * f * w[pd];
                     }
                 }
@@ -133,13 +146,15 @@ __global__ __launch_bounds__(QKN_MAX_WAVES * BN_WAVE) void qk_norm_store_kernel(
             if (!a.v_pages) continue;
             const int kvh = head - a.H - a.Hkv;
             const T* v = a.v_from_k ? row + (size_t)(a.H + kvh) * a.hs : row + (size_t)(a.H + a.Hkv) * a.hs + (size_t)kvh * a.vd;
+            const float* bias = a.bias && a.v_from_k ? a.bias + (size_t)(a.H + kvh) * a.hs : nullptr;
             const int page = a.block_table[(size_t)a.seq_index[t] * a.bt_stride + pos / BN_PAGE];
             if (a.v_transposed) {
                 T* dst = reinterpret_cast<T*>(a.v_pages) + ((size_t)page * a.Hkv + kvh) * a.vd * BN_PAGE + pos % BN_PAGE;
-                for (int d = lane; d < a.vd; d += BN_WAVE) dst[(size_t)d * BN_PAGE] = v[d];
+                for (int d = lane; d < a.vd; d += BN_WAVE)
+                    dst[(size_t)d * BN_PAGE] = bias ? from_f32<T>(to_f32(v[d]) + bias[d]) : v[d];
             } else {
                 T* dst = reinterpret_cast<T*>(a.v_pages) + (((size_t)page * a.Hkv + kvh) * BN_PAGE + pos % BN_PAGE) * a.vd;
-                for (int d = lane; d < a.vd; d += BN_WAVE) dst[d] = v[d];
+                for (int d = lane; d < a.vd; d += BN_WAVE) dst[d] = bias ? from_f32<T>(to_f32(v[d]) + bias[d]) : v[d];
             }
         }
     }
@@ -149,7 +164,7 @@ extern "C" int bn_qk_norm_store(int dtype, void* qkv, int ld, const int* positio
                                 const int* block_table, int bt_stride, void* k_pages, void* v_pages, const float* wq,
                                 const float* wk, int n_tokens, int H, int Hkv, int hs, int vd, float eps, float temp_coef,
                                 int temp_every, int v_transposed, int norm_all, const float* inv_freq, int rope_dims,
-                                int rope_interleaved, int v_from_k, hipStream_t s) {
+                                int rope_interleaved, int v_from_k, const float* bias, const float* head_temp, hipStream_t s) {
     if (n_tokens <= 0 || H <= 0 || Hkv <= 0 || hs <= 0 || hs > BN_MAX_HEAD_DIM || vd <= 0 || !qkv || !positions) return BN_ERR_ARG;
     if ((k_pages == nullptr) != (v_pages == nullptr) || (k_pages && (!seq_index || !block_table))) return BN_ERR_ARG;
     if ((wq == nullptr) != (wk == nullptr) || ld < H * hs + Hkv * (v_from_k ? hs : hs + vd) || (v_from_k && vd != hs)) return BN_ERR_ARG;
@@ -160,7 +175,7 @@ extern "C" int bn_qk_norm_store(int dtype, void* qkv, int ld, const int* positio
     a.ld = ld; a.bt_stride = bt_stride; a.H = H; a.Hkv = Hkv; a.hs = hs; a.vd = vd;
     a.eps = eps; a.temp_coef = temp_coef; a.temp_every = temp_every; a.v_transposed = v_transposed ? 1 : 0;
     a.norm_all = norm_all ? 1 : 0; a.rope_dims = inv_freq ? rope_dims : 0; a.rope_interleaved = rope_interleaved ? 1 : 0;
-    a.v_from_k = v_from_k ? 1 : 0;
+    a.v_from_k = v_from_k ? 1 : 0; a.bias = bias; a.head_temp = head_temp;
     const int n_heads = H + 2 * Hkv;
     const int waves = norm_all ? (n_heads < QKN_MAX_WAVES ? (n_heads < QKN_WAVES ? QKN_WAVES : n_heads) : QKN_MAX_WAVES) : QKN_WAVES;
     const dim3 grid(n_tokens, norm_all ? 1 : (n_heads + QKN_WAVES - 1) / QKN_WAVES), block(waves * BN_WAVE);

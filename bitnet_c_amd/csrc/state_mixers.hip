@@ -35,23 +35,28 @@ __device__ __forceinline__ SeqRange seq_range(const int* tiles, const int* seq_l
 
 // ---- token shift ----------------------------------------------------------------------------------------------------
 // out[s, t, :] for s < n_mix.  The previous row of the flattened batch is the previous token when it belongs to the same
-// sequence; else the sequence's state holds it (zero at position 0).  The state is read only: the recurrence's
-// kernel stores the step's last h afterwards, when every reader is done.
-template <typename T>
-__global__ void token_shift_kernel(T* __restrict__ out, const T* __restrict__ h, const float* __restrict__ mu,
-                                   const float* __restrict__ state, size_t state_stride, const int* __restrict__ positions,
-                                   const int* __restrict__ seq_index, const int* __restrict__ slot_ids, int T_rows, int D,
-                                   int n_mix) {
+// sequence; else the sequence's state holds it (zero at position 0).  seq_lens null: the state is read only, and the
+// recurrence's kernel stores the step's last h afterwards, when every reader is done.  Else (seq_lens: the sequences'
+// lengths behind the step) the workgroup of a sequence's first row, the only reader of the sequence's state, stores the
+// step's last row there, each thread the elements that it has read.  TI: the type of h; TO: of the mixes.
+template <typename TI, typename TO>
+__global__ void token_shift_kernel(TO* __restrict__ out, const TI* __restrict__ h, const float* __restrict__ mu,
+                                   float* state, size_t state_stride, const int* __restrict__ positions,
+                                   const int* __restrict__ seq_index, const int* __restrict__ slot_ids,
+                                   const int* __restrict__ seq_lens, int T_rows, int D, int n_mix) {
     const int t = blockIdx.x;
     const int pos = positions[t], seq = seq_index[t];
     const int before = t > 0 ? t - 1 : 0;
     const int pos_b = positions[before], seq_b = seq_index[before], slot = slot_ids[seq];     // all asked for together
-    const T* cur = h + (size_t)t * D;
+    const TI* cur = h + (size_t)t * D;
     const bool inside = t > 0 && pos > 0 && seq_b == seq && pos_b == pos - 1;
     // both candidates for the previous row are loaded, from places that exist, and one is chosen: a load under a
     // branch would be waited for where it stands, element after element
-    const T* prev_row = h + (size_t)(inside ? t - 1 : t) * D;
-    const float* prev_state = state + (size_t)slot * state_stride;
+    const TI* prev_row = h + (size_t)(inside ? t - 1 : t) * D;
+    float* prev_state = state + (size_t)slot * state_stride;
+    const bool keeps = seq_lens && pos >= 0 && !inside;           // the first row of its sequence in this step
+    const int last = keeps ? min(t + max(seq_lens[seq] - 1 - pos, 0), T_rows - 1) : t;
+    const TI* last_row = h + (size_t)last * D;
 #pragma unroll 4
     for (int e = threadIdx.x; e < D; e += blockDim.x) {
         const float c = to_f32(cur[e]);
@@ -59,23 +64,75 @@ __global__ void token_shift_kernel(T* __restrict__ out, const T* __restrict__ h,
         const float p = inside ? pr : (pos > 0 ? ps : 0.f);
         const float d = p - c;
         for (int s = 0; s < n_mix; ++s)
-            out[((size_t)s * T_rows + t) * D + e] = from_f32<T>(pos >= 0 ? fmaf(d, mu[(size_t)s * D + e], c) : 0.f);
+            out[((size_t)s * T_rows + t) * D + e] = from_f32<TO>(pos >= 0 ? fmaf(d, mu[(size_t)s * D + e], c) : 0.f);
+        if (keeps) prev_state[e] = to_f32(last_row[e]);
     }
 }
 
-extern "C" int bn_token_shift(int dtype, void* out, const void* h, const float* mu, const float* state,
+// The same for one mix of a float32 stream, four elements a thread (D a multiple of 4, everything 16-byte aligned): what a
+// block that mixes its stream with the previous token's runs over a whole prompt step.
+template <typename TO>
+__global__ __launch_bounds__(256) void token_shift_stream_kernel(TO* __restrict__ out, const float* __restrict__ x,
+                                                                 const float* __restrict__ mu, float* state, size_t state_stride,
+                                                                 const int* __restrict__ positions, const int* __restrict__ seq_index,
+                                                                 const int* __restrict__ slot_ids, const int* __restrict__ seq_lens,
+                                                                 int T_rows, int D) {
+    const int t = blockIdx.x;
+    const int pos = positions[t], seq = seq_index[t];
+    const int before = t > 0 ? t - 1 : 0;
+    const int pos_b = positions[before], seq_b = seq_index[before], slot = slot_ids[seq];
+    const bool inside = t > 0 && pos > 0 && seq_b == seq && pos_b == pos - 1;
+    float* st = state + (size_t)slot * state_stride;
+    const float* cur = x + (size_t)t * D;
+    const float* prev = inside ? cur - D : st;                    // one load for either candidate
+    const bool has_prev = pos > 0, keeps = pos >= 0 && !inside;
+    const int last = keeps ? min(t + max(seq_lens[seq] - 1 - pos, 0), T_rows - 1) : t;
+    const float* last_row = x + (size_t)last * D;
+    TO* o = out + (size_t)t * D;
+    for (int e = threadIdx.x * 4; e < D; e += 1024) {
+        const float4 c = *reinterpret_cast<const float4*>(cur + e), m = *reinterpret_cast<const float4*>(mu + e);
+        float4 p = *reinterpret_cast<const float4*>(prev + e);
+        if (!has_prev) p = make_float4(0.f, 0.f, 0.f, 0.f);
+        float4 r;
+        r.x = fmaf(p.x - c.x, m.x, c.x); r.y = fmaf(p.y - c.y, m.y, c.y);
+        r.z = fmaf(p.z - c.z, m.z, c.z); r.w = fmaf(p.w - c.w, m.w, c.w);
+        if (pos < 0) r = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (sizeof(TO) == 2) {
+            bf16 b[4] = {from_f32<bf16>(r.x), from_f32<bf16>(r.y), from_f32<bf16>(r.z), from_f32<bf16>(r.w)};
+            *reinterpret_cast<uint2*>(o + e) = *reinterpret_cast<const uint2*>(b);
+        } else {
+            *reinterpret_cast<float4*>(o + e) = r;
+        }
+        if (keeps) *reinterpret_cast<float4*>(st + e) = *reinterpret_cast<const float4*>(last_row + e);
+    }
+}
+
+// in_dtype: of h; dtype: of the mixes (in_dtype equal to it, or float32).  seq_lens: see above.
+extern "C" int bn_token_shift(int in_dtype, int dtype, void* out, const void* h, const float* mu, float* state,
                               long long state_stride, const int* positions, const int* seq_index, const int* slot_ids,
-                              int n_tokens, int D, int n_mix, hipStream_t s) {
+                              const int* seq_lens, int n_tokens, int D, int n_mix, hipStream_t s) {
     if (n_tokens <= 0 || D <= 0 || n_mix <= 0 || !out || !h || !mu || !state || !positions || !seq_index || !slot_ids)
         return BN_ERR_ARG;
-    if (dtype == BN_DT_F32)
-        hipLaunchKernelGGL(token_shift_kernel<float>, dim3(n_tokens), dim3(256), 0, s, (float*)out, (const float*)h, mu, state,
-                           (size_t)state_stride, positions, seq_index, slot_ids, n_tokens, D, n_mix);
-    else if (dtype == BN_DT_BF16)
-        hipLaunchKernelGGL(token_shift_kernel<bf16>, dim3(n_tokens), dim3(256), 0, s, (bf16*)out, (const bf16*)h, mu, state,
-                           (size_t)state_stride, positions, seq_index, slot_ids, n_tokens, D, n_mix);
+    if ((dtype != BN_DT_F32 && dtype != BN_DT_BF16) || (in_dtype != dtype && in_dtype != BN_DT_F32)) return BN_ERR_DTYPE;
+    const dim3 grid(n_tokens), block(256);
+    const size_t st = (size_t)state_stride;
+    if (in_dtype == BN_DT_F32 && seq_lens && n_mix == 1 && D % 4 == 0 && st % 4 == 0 &&
+        !(((uintptr_t)out | (uintptr_t)h | (uintptr_t)mu | (uintptr_t)state) & 15)) {
+        if (dtype == BN_DT_F32)
+            hipLaunchKernelGGL(token_shift_stream_kernel<float>, grid, block, 0, s, (float*)out, (const float*)h, mu, state, st,
+                               positions, seq_index, slot_ids, seq_lens, n_tokens, D);
+        else
+            hipLaunchKernelGGL(token_shift_stream_kernel<bf16>, grid, block, 0, s, (bf16*)out, (const float*)h, mu, state, st,
+                               positions, seq_index, slot_ids, seq_lens, n_tokens, D);
+    } else if (in_dtype == BN_DT_F32 && dtype == BN_DT_F32)
+        hipLaunchKernelGGL((token_shift_kernel<float, float>), grid, block, 0, s, (float*)out, (const float*)h, mu, state, st,
+                           positions, seq_index, slot_ids, seq_lens, n_tokens, D, n_mix);
+    else if (in_dtype == BN_DT_F32)
+        hipLaunchKernelGGL((token_shift_kernel<float, bf16>), grid, block, 0, s, (bf16*)out, (const float*)h, mu, state, st,
+                           positions, seq_index, slot_ids, seq_lens, n_tokens, D, n_mix);
     else
-        return BN_ERR_DTYPE;
+        hipLaunchKernelGGL((token_shift_kernel<bf16, bf16>), grid, block, 0, s, (bf16*)out, (const bf16*)h, mu, state, st,
+                           positions, seq_index, slot_ids, seq_lens, n_tokens, D, n_mix);
     return bn_launch_status();
 }
 

@@ -49,6 +49,7 @@ class DecoderModel:
         self.final_norm = NORMS.build(plan.final_norm) if plan.final_norm is not None else None
         self.lm_head_bias = None         # [V] float32, when the plan names one
         self.position_freq = None        # [ceil(D / 2)] float32: the frequencies of a sinusoidal position vector, when the plan has one
+        self.position_table = None       # [max positions, D] in the compute dtype: learned position vectors, when the plan names them
         self.embedding = None            # [V, D] in the compute dtype
         self.lm_head = None              # [V, D]; the embedding itself when tied
 
@@ -71,6 +72,9 @@ class DecoderModel:
             done([p.lm_head_bias_name])
         if p.position_sinusoid_base > 0:
             self.position_freq = ops.sinusoid_frequencies(p.hidden_size, p.position_sinusoid_base).to(self.device)
+        if p.position_table_name is not None:
+            self.position_table = upload(tensors[p.position_table_name], self.device, self.dtype)
+            done([p.position_table_name])
         self.embedding = upload(tensors[p.embedding_name], self.device, self.dtype)
         done([p.embedding_name])
         if p.lm_head_name is None:
@@ -176,6 +180,9 @@ class DecoderModel:
         if self.position_freq is not None:
             x = ops.embed_gather_sinusoid(self.embedding, ctx.tokens, ctx.positions, self.position_freq,
                                           self.plan.embedding_multiplier)
+        elif self.position_table is not None:
+            x = ops.embed_gather_learned(self.embedding, ctx.tokens, ctx.positions, self.position_table,
+                                         self.plan.embedding_multiplier)
         else:
             x = ops.embed_gather(self.embedding, ctx.tokens, self.plan.embedding_multiplier)    # src/model_embed.c:6-28
         if self.plan.residual_streams > 0:

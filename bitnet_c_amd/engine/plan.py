@@ -49,6 +49,9 @@ class ModelPlan:
     # Positions that enter with the embedding instead of inside the mixers: > 0 adds a sinusoidal vector to every
     # embedding row, entry 2i = sin(p base^(-2i/hidden)), entry 2i + 1 = cos of the same angle.
     position_sinusoid_base: float = 0.0
+    # Or a learned vector per position, added to the embedding's rows (not multiplied by the embedding's constant): the
+    # name of a tensor [max_positions, hidden]; None: none.
+    position_table_name: Optional[str] = None
     logit_scale: float = 1.0             # the logits times this (before a bias or a soft-cap)
     # > 0: the residual is that many float32 streams (parts/hyper.py: HyperStream, read and written by "hyper" blocks) that
     # all start as the embedding's rows and are summed in front of the final norm; 0: the one stream of the other blocks.
@@ -60,6 +63,9 @@ class ModelPlan:
         if self.position_sinusoid_base < 0 or self.position_sinusoid_base == 1 or not self.logit_scale > 0:
             raise ValueError("the base of a sinusoidal position vector is 0 (none) or a positive number other than 1, "
                              "and the logits' multiplier is positive")
+        if self.position_table_name is not None and (self.max_positions < 1 or self.position_sinusoid_base > 0):
+            raise ValueError("a table of position vectors has a row for each of max_positions positions, and no sinusoidal "
+                             "vector beside it")
         if self.residual_streams < 0:
             raise ValueError("the number of residual streams is 0 (the plain residual) or positive")
         for i, e in enumerate(self.schedule):
@@ -96,6 +102,8 @@ class ModelPlan:
                 put(self.final_norm_names[local], spec.shape, spec.init, spec.optional)
         if self.lm_head_name is not None:
             put(self.lm_head_name, (self.vocab_size, self.hidden_size), "normal")
+        if self.position_table_name is not None:
+            put(self.position_table_name, (self.max_positions, self.hidden_size), "normal")
         if self.lm_head_bias_name is not None:
             put(self.lm_head_bias_name, (self.vocab_size,), "normal")
         return out

@@ -46,16 +46,22 @@ _SIGNATURES = {
         "bn_bias_add": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
         "bn_embed_gather_sinusoid": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float,
                                      c_void_p],
+        "bn_embed_gather_learned": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_float,
+                                    c_void_p],
         "bn_unary_act_apply": [c_int, c_void_p, c_void_p, c_longlong, c_int, c_void_p],
         "bn_scale": [c_void_p, c_longlong, c_float, c_void_p],
         "bn_rmsnorm_mean": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p],
         "bn_add_normed_rmsnorm": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int,
                                   c_float, c_void_p],
     },
+    "post_norm": {
+        "bn_post_norm": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_float, c_void_p, c_int, c_int,
+                         c_void_p, c_void_p, c_longlong, c_void_p, c_void_p, c_void_p],
+    },
     "qk_norm": {
         "bn_qk_norm_store": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                              c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_int, c_void_p, c_int,
-                             c_int, c_int, c_void_p],
+                             c_int, c_int, c_void_p, c_void_p, c_void_p],
     },
     "latent": {
         "bn_latent_store": [c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
@@ -78,10 +84,11 @@ _SIGNATURES = {
     "attn_mfma_general": {
         "bn_attn_general_supports": [c_int, c_int],
         "bn_attn_general_prompt": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int,
-                                   c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p],
+                                   c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
+                                   c_void_p],
         "bn_attn_general_decode": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int,
-                                   c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p,
-                                   c_void_p, c_void_p, c_void_p],
+                                   c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
+                                   c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     },
     "hyper": {
         "bn_hc_step": [c_int, c_int, c_void_p, c_longlong, c_void_p, c_longlong, c_void_p, c_int, c_longlong, c_void_p, c_void_p,
@@ -112,8 +119,8 @@ _SIGNATURES = {
         "bn_row_norm_gate": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_int, c_void_p],
     },
     "state_mixers": {
-        "bn_token_shift": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p, c_void_p, c_void_p, c_int,
-                           c_int, c_int, c_void_p],
+        "bn_token_shift": [c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p, c_void_p, c_void_p, c_void_p,
+                           c_int, c_int, c_int, c_void_p],
         "bn_wkv_supports": [c_int, c_int],
         "bn_wkv_state_floats": [c_int, c_int],
         "bn_wkv_scan": [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
@@ -135,7 +142,7 @@ _SIGNATURES = {
         "bn_attn_rows_key_tile": [c_int, c_int],
         "bn_attn_rows": [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                          c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
-                         c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p],
+                         c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p],
     },
     "attn_mfma": {
         "bn_attn_mfma_supports": [c_int],
@@ -1232,12 +1239,38 @@ def _sink_args(sink, H: int, what: str):
     return 1, sink.data_ptr()
 
 
+def _distance_args(distance_bias, H: int, what: str):
+    """Addresses of the two vectors of a distance bias as the kernels take them: None, no bias; (a, b), a logarithmic one;
+    (a, None), a linear one."""
+    if distance_bias is None:
+        return None, None
+    a, b = distance_bias
+    for t, nm in ((a, "distance_bias[0]"), (b, "distance_bias[1]")):
+        if t is None and nm.endswith("[1]"):
+            continue
+        _dev(t, nm, torch.float32, 1)
+        if t.numel() != H or not t.is_contiguous():
+            raise KernelError(f"{what}: {nm} must hold one float32 per head")
+    return a.data_ptr(), b.data_ptr() if b is not None else None
+
+
+def _gate_args(gate, T: int, width: int, what: str):
+    """(address, row stride) of a gate [T, width] (a run of columns of a wider tensor will do), or (None, 0)."""
+    if gate is None:
+        return None, 0
+    _dev(gate, "gate", torch.bfloat16, 2)
+    ld = _rows(gate, "gate")
+    if tuple(gate.shape) != (T, width) or ld % 4 or gate.data_ptr() % 8:
+        raise KernelError(f"{what}: gate {tuple(gate.shape)} (row stride {ld}) is not [{T}, {width}] with 8-byte aligned rows")
+    return gate.data_ptr(), ld
+
+
 def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
               block_table: torch.Tensor, H: int, Hkv: int, hs: int, scale: float, *, window: int = 0,
               tiles=None, qt: int = 0, seq_lens=None, n_splits: int = 1, chunk: int = 0,
               force_vector: bool = False, fused_rotate=None, fused_write: bool = False, by_length=None,
               max_len_dev=None, v_transposed=None, row_scale: Optional["DeferredNorm"] = None, blocked=None,
-              v_dim: int = 0, distance_bias=None, sink: bool = False) -> None:
+              v_dim: int = 0, distance_bias=None, sink: bool = False, keep_first: int = 0) -> None:
     """Causal attention of the (rotated) Q heads in qkv over the paged cache.
 
     Prompt form: `tiles` [n, 4] int32 = (sequence, first token row, tokens (<= qt), position of
@@ -1266,7 +1299,8 @@ def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pag
     value of every row by it.
     What only the vector kernel does (pages that are not blocked): v_dim, value heads of another width than the keys'
     (out is then [T, H * v_dim]); distance_bias = (a, b), two float32 tensors [H]: a[h] * ln(1 + b[h] * (i - j)) is taken
-    off the score of query position i and key position j; sink: the softmax has one more term without a value: True, of
+    off the score of query position i and key position j, or, with (a, None), a[h] * (i - j); keep_first: with a window, the
+    first keep_first positions stay visible however far back they are; sink: the softmax has one more term without a value: True, of
     score 0 (1 is added to its denominator); a float32 tensor [H], of that score per head (exp(sink[h]) is added)."""
     require_gpu()
     _dev(qkv, "qkv", dims=2)
@@ -1281,17 +1315,13 @@ def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pag
     if vd % 2 or vd < 2 or vd > MAX_HEAD_DIM:
         raise KernelError(f"attention: value width {vd} is not supported (even, at most {MAX_HEAD_DIM})")
     sink_flag, sink_ptr = _sink_args(sink, H, "attention")
-    extras = vd != hs or distance_bias is not None or bool(sink_flag)
+    extras = vd != hs or distance_bias is not None or bool(sink_flag) or keep_first != 0
+    if keep_first < 0:
+        raise KernelError(f"attention: keep_first {keep_first}")
     if extras and layout == "blocked":
-        raise KernelError("attention: another value width, a distance bias and a sink are the vector kernel's, which reads "
+        raise KernelError("attention: another value width, a distance bias, kept first positions and a sink are the vector kernel's, which reads "
                           "pages with a row per position or transposed values")
-    da = db = None
-    if distance_bias is not None:
-        da, db = distance_bias
-        for t, nm in ((da, "distance_bias[0]"), (db, "distance_bias[1]")):
-            _dev(t, nm, torch.float32, 1)
-            if t.numel() != H or not t.is_contiguous():
-                raise KernelError(f"attention: {nm} must hold one float32 per head")
+    da, db = _distance_args(distance_bias, H, "attention")
     if hs % 2 or hs < 2 or hs > MAX_HEAD_DIM:
         raise KernelError(f"attention: head size {hs} is not supported (even, at most {MAX_HEAD_DIM})")
     if not block_table.is_contiguous():
@@ -1389,8 +1419,7 @@ def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pag
         k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(), block_table.shape[1],
         sl, tl, n_tiles, T, H, Hkv, hs, RT, GT, int(window), float(scale), int(n_splits), int(chunk),
         po, pm, int(vt), max_len_dev.data_ptr() if max_len_dev is not None else None, int(fold), vd,
-        da.data_ptr() if da is not None else None, db.data_ptr() if db is not None else None, sink_flag, sink_ptr, _stream()),
-        "attention")
+        da, db, sink_flag, sink_ptr, int(keep_first), _stream()), "attention")
 
 
 
@@ -1402,7 +1431,7 @@ def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
                   q_weight=None, k_weight=None, eps: float = 0.0, temp_coef: float = 0.0, temp_every: int = 0,
                   seq_index=None, block_table=None, k_pages=None, v_pages=None, v_transposed: bool = False,
                   norm_projection: bool = False, inv_freq=None, rope_dims: int = 0, rope_interleaved: bool = False,
-                  v_from_k: bool = False) -> None:
+                  v_from_k: bool = False, bias=None, head_temp=None) -> None:
     """In place on qkv [T, H hs + Hkv (hs + v_dim)]: every query and key head under an RMSNorm of its own (weights
     [hs] float32, shared by the heads; both or neither), or, with norm_projection, one RMSNorm over the whole query
     projection and one over the whole key projection (weights [H hs] and [Hkv hs]); then the first rope_dims dimensions
@@ -1411,7 +1440,9 @@ def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
     1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p (temp_every 0: no temperature); the keys and the
     values go into the pages when pages are given (keys a row per position; values the same way, or transposed inside a
     page when v_transposed).  Rows with position < 0 are left alone.  v_from_k: the values are the key projections as
-    they arrived (before norm and rotation); qkv is [T, (H + Hkv) hs] then and v_dim equals hs."""
+    they arrived (before norm and rotation; with their bias); qkv is [T, >= (H + Hkv) hs] then and v_dim equals hs.  bias [(H + Hkv) hs]
+    float32: added to the query and key projections before anything else; head_temp [H] float32: multiplies the finished
+    queries of each head (columns behind the heads, a gate's say, are left alone)."""
     require_gpu()
     _dev(qkv, "qkv", dims=2)
     _dev(positions, "positions", torch.int32, 1)
@@ -1434,6 +1465,11 @@ def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
         _dev(inv_freq, "inv_freq", torch.float32, 1)
         if rope_dims <= 0 or rope_dims % 2 or rope_dims > hs or inv_freq.numel() != rope_dims // 2 or not inv_freq.is_contiguous():
             raise KernelError(f"qk_norm_store: rope_dims {rope_dims} does not fit hs={hs} / inv_freq {tuple(inv_freq.shape)}")
+    for t, nm, n in ((bias, "bias", (H + Hkv) * hs), (head_temp, "head_temp", H)):
+        if t is not None:
+            _dev(t, nm, torch.float32, 1)
+            if t.numel() != n or not t.is_contiguous():
+                raise KernelError(f"qk_norm_store: {nm} must hold {n} float32 values")
     if k_pages is not None:
         _check_pages(k_pages, v_pages, Hkv, hs, qkv.dtype, bool(v_transposed), False, vd)
         _dev(seq_index, "seq_index", torch.int32, 1)
@@ -1450,7 +1486,8 @@ def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
         k_weight.data_ptr() if k_weight is not None else None, T, H, Hkv, hs, vd, float(eps), float(temp_coef),
         int(temp_every), int(bool(v_transposed)), int(bool(norm_projection)),
         inv_freq.data_ptr() if inv_freq is not None else None, int(rope_dims), int(bool(rope_interleaved)),
-        int(bool(v_from_k)), _stream()), "qk_norm_store")
+        int(bool(v_from_k)), bias.data_ptr() if bias is not None else None,
+        head_temp.data_ptr() if head_temp is not None else None, _stream()), "qk_norm_store")
 
 
 GENERAL_PROMPT_TILE = 16       # query tokens of a tile of attention_general_prompt
@@ -1467,10 +1504,11 @@ def attention_general_supported(dtype, hs: int, v_dim: int) -> bool:
 
 def attention_general_prompt(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                              block_table: torch.Tensor, H: int, Hkv: int, hs: int, v_dim: int, scale: float, tiles: torch.Tensor,
-                             *, distance_bias=None, sink: bool = False, window: int = 0) -> None:
+                             *, distance_bias=None, sink: bool = False, window: int = 0, keep_first: int = 0, gate=None) -> None:
     """Causal prompt attention on the matrix cores for what attention() leaves to the vector kernel: bf16, keys 32, 64,
     96, 128 or 256 wide, values of a width of their own from the same list, a distance bias and a sink (as attention()'s),
-    a window (> 0: a query sees the last `window` positions, its own included).  qkv's row stride is a multiple of 8.
+    a window (> 0: a query sees the last `window` positions, its own included, and the first keep_first positions).  gate: a
+    bf16 tensor [T, H v_dim] (it may be columns of a wider one): the result times sigmoid(gate).  qkv's row stride is a multiple of 8.
     Pages: keys a row per position, values transposed.  tiles [n, 4] int32: (sequence, first row, rows <= 16, position of
     the first), any order, tiles of no rows skipped.  out [T, H v_dim]."""
     require_gpu()
@@ -1486,22 +1524,17 @@ def attention_general_prompt(qkv: torch.Tensor, out: torch.Tensor, k_pages: torc
             or not tiles.is_contiguous() or not block_table.is_contiguous()):
         raise KernelError(f"attention_general_prompt: qkv {tuple(qkv.shape)} / out {tuple(out.shape)} / tiles {tuple(tiles.shape)} "
                           f"do not fit H={H} hs={hs} v_dim={v_dim}")
-    da = db = None
-    if distance_bias is not None:
-        da, db = distance_bias
-        for t, nm in ((da, "distance_bias[0]"), (db, "distance_bias[1]")):
-            _dev(t, nm, torch.float32, 1)
-            if t.numel() != H or not t.is_contiguous():
-                raise KernelError(f"attention_general_prompt: {nm} must hold one float32 per head")
-    if window < 0 or _rows(qkv, "qkv") % 8 or qkv.data_ptr() % 16:
+    da, db = _distance_args(distance_bias, H, "attention_general_prompt")
+    gp, gld = _gate_args(gate, T, H * v_dim, "attention_general_prompt")
+    if window < 0 or keep_first < 0 or _rows(qkv, "qkv") % 8 or qkv.data_ptr() % 16:
         raise KernelError(f"attention_general_prompt: window {window} / row stride {_rows(qkv, 'qkv')} (a multiple of 8, 16-byte aligned)")
     if T == 0 or tiles.shape[0] == 0:
         return
     _check(_fn("attn_mfma_general", "bn_attn_general_prompt")(
         qkv.data_ptr(), _rows(qkv, "qkv"), out.data_ptr(), H * v_dim, k_pages.data_ptr(), v_pages.data_ptr(),
         block_table.data_ptr(), block_table.shape[1], tiles.data_ptr(), tiles.shape[0], H, Hkv, hs, v_dim, float(scale),
-        da.data_ptr() if da is not None else None, db.data_ptr() if db is not None else None,
-        *_sink_args(sink, H, "attention_general_prompt"), int(window), _stream()), "attention_general_prompt")
+        da, db, *_sink_args(sink, H, "attention_general_prompt"), int(window), int(keep_first), gp, gld, _stream()),
+        "attention_general_prompt")
 
 
 def general_decode_plan(n_seqs: int, H: int, Hkv: int, max_len: int, window: int = 0):
@@ -1519,13 +1552,14 @@ def general_decode_plan(n_seqs: int, H: int, Hkv: int, max_len: int, window: int
 def attention_general_decode(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                              block_table: torch.Tensor, seq_lens: torch.Tensor, H: int, Hkv: int, hs: int, v_dim: int, scale: float,
                              *, window: int = 0, n_splits: int = 1, chunk: int = 0, max_len_dev=None, distance_bias=None,
-                             sink: bool = False) -> None:
+                             sink: bool = False, keep_first: int = 0, gate=None) -> None:
     """The decode form of attention_general_prompt (bf16, the same head sizes and pages): row b of qkv is sequence b's new
     token, seq_lens [B] its keys in the cache (0: a padding row, whose output is zeros).  A wave takes the heads that share
     a kv head together, so their keys and values are read once.  n_splits > 1 cuts the keys into runs of `chunk` positions
     (a multiple of PAGE; with max_len_dev, a device int32, into runs of split_chunk(longest sequence, n_splits)), merged in
     index order; with a window the runs are counted from the page of the window's first key and need only cover
-    window + PAGE positions.  distance_bias, sink: as attention()'s."""
+    window + PAGE positions (kept first keys are the first run's).  distance_bias, sink, keep_first: as attention()'s; gate: as
+    attention_general_prompt's."""
     require_gpu()
     _dev(qkv, "qkv", torch.bfloat16, 2)
     _dev(out, "out", torch.bfloat16, 2)
@@ -1539,15 +1573,10 @@ def attention_general_decode(qkv: torch.Tensor, out: torch.Tensor, k_pages: torc
             or block_table.shape[0] < T or not block_table.is_contiguous() or not seq_lens.is_contiguous()):
         raise KernelError(f"attention_general_decode: qkv {tuple(qkv.shape)} / out {tuple(out.shape)} / seq_lens "
                           f"{tuple(seq_lens.shape)} do not fit H={H} hs={hs} v_dim={v_dim}")
-    if window < 0 or _rows(qkv, "qkv") % 8 or qkv.data_ptr() % 16:
+    if window < 0 or keep_first < 0 or _rows(qkv, "qkv") % 8 or qkv.data_ptr() % 16:
         raise KernelError(f"attention_general_decode: window {window} / row stride {_rows(qkv, 'qkv')} (a multiple of 8, 16-byte aligned)")
-    da = db = None
-    if distance_bias is not None:
-        da, db = distance_bias
-        for t, nm in ((da, "distance_bias[0]"), (db, "distance_bias[1]")):
-            _dev(t, nm, torch.float32, 1)
-            if t.numel() != H or not t.is_contiguous():
-                raise KernelError(f"attention_general_decode: {nm} must hold one float32 per head")
+    da, db = _distance_args(distance_bias, H, "attention_general_decode")
+    gp, gld = _gate_args(gate, T, H * v_dim, "attention_general_decode")
     part_o = part_ml = None
     if n_splits > 1:
         if max_len_dev is not None:
@@ -1567,8 +1596,7 @@ def attention_general_decode(qkv: torch.Tensor, out: torch.Tensor, k_pages: torc
     _check(_fn("attn_mfma_general", "bn_attn_general_decode")(
         qkv.data_ptr(), _rows(qkv, "qkv"), out.data_ptr(), H * v_dim, k_pages.data_ptr(), v_pages.data_ptr(),
         block_table.data_ptr(), block_table.shape[1], seq_lens.data_ptr(), T, H, Hkv, hs, v_dim, float(scale),
-        da.data_ptr() if da is not None else None, db.data_ptr() if db is not None else None,
-        *_sink_args(sink, H, "attention_general_decode"), int(window), int(n_splits), int(chunk), part_o.data_ptr() if part_o is not None else None,
+        da, db, *_sink_args(sink, H, "attention_general_decode"), int(window), int(keep_first), gp, gld, int(n_splits), int(chunk), part_o.data_ptr() if part_o is not None else None,
         part_ml.data_ptr() if part_ml is not None else None,
         max_len_dev.data_ptr() if (max_len_dev is not None and n_splits > 1) else None, _stream()), "attention_general_decode")
 
@@ -1633,6 +1661,82 @@ def embed_gather_sinusoid(table: torch.Tensor, tokens: torch.Tensor, positions: 
     return x
 
 
+def embed_gather_learned(table: torch.Tensor, tokens: torch.Tensor, positions: torch.Tensor, pos_table: torch.Tensor,
+                         scale: float = 1.0) -> torch.Tensor:
+    """embed_gather plus the row of pos_table [max positions, D] at each token's position (not scaled); a row with
+    position < 0 gets none."""
+    require_gpu()
+    _dev(table, "table", dims=2)
+    _dev(tokens, "tokens", torch.int32, 1)
+    _dev(positions, "positions", torch.int32, 1)
+    _dev(pos_table, "pos_table", table.dtype, 2)
+    n, dim = tokens.numel(), table.shape[1]
+    if (not table.is_contiguous() or not tokens.is_contiguous() or not positions.is_contiguous() or positions.numel() != n
+            or pos_table.shape[1] != dim or not pos_table.is_contiguous()):
+        raise KernelError("embed_gather_learned: contiguous inputs, a position per token and position rows as wide as the embedding's")
+    x = torch.empty((n, dim), dtype=torch.float32, device=table.device)
+    if n:
+        _check(_fn("elementwise", "bn_embed_gather_learned")(
+            _code(table.dtype), x.data_ptr(), table.data_ptr(), tokens.data_ptr(), positions.data_ptr(), pos_table.data_ptr(),
+            n, dim, table.shape[0], pos_table.shape[0], float(scale), _stream()), "embed_gather_learned")
+    return x
+
+
+def post_norm(x: torch.Tensor, delta, gain: Optional[torch.Tensor], alpha: float, weight: torch.Tensor, eps: float, *,
+              out_dtype=None, mu: Optional[torch.Tensor] = None, state: Optional[torch.Tensor] = None, positions=None,
+              slot_ids=None) -> Optional[torch.Tensor]:
+    """The float32 stream x [T, D], in place: x <- weight * v / sqrt(mean(v^2) + eps) with v = alpha x + gain * delta (delta: a
+    tensor or PartialSums; gain [D] float32, None: 1).  out_dtype: the new rows are also returned in that type.  mu [D] (a
+    decode step, row b the one new token of sequence b): the rows returned are x + (x' - x) * mu with x' the first D values of
+    the sequence's state row (zeros at position 0), which then take the new x; rows with position < 0 touch no state."""
+    require_gpu()
+    _dev(x, "x", torch.float32, 2)
+    T, D = x.shape
+    for t, nm in ((weight, "weight"), (gain, "gain"), (mu, "mu")):
+        if t is not None:
+            _dev(t, nm, torch.float32, 1)
+            if t.numel() != D or not t.is_contiguous():
+                raise KernelError(f"post_norm: {nm} must hold {D} float32 values")
+    parts = isinstance(delta, PartialSums)
+    y = delta.slabs if parts else delta
+    _dev(y, "delta")
+    if not x.is_contiguous() or tuple(delta.shape) != (T, D) or not y.is_contiguous():
+        raise KernelError(f"post_norm: x {tuple(x.shape)} and delta {tuple(delta.shape)} must be contiguous and alike")
+    kind = out_dtype or (torch.bfloat16 if parts else y.dtype)
+    if not parts and y.dtype != kind:
+        raise KernelError(f"post_norm: delta in {y.dtype} and rows in {kind}")
+    stride, sp, pp, ip = 0, None, None, None
+    if mu is not None:
+        if out_dtype is None:
+            raise KernelError("post_norm: mixing with the previous row needs an output type")
+        stride = _state_rows(state, D, "post_norm")
+        for t, nm in ((positions, "positions"), (slot_ids, "slot_ids")):
+            _dev(t, nm, torch.int32, 1)
+            if t.numel() != T or not t.is_contiguous():
+                raise KernelError(f"post_norm: {nm} has one entry per row")
+        sp, pp, ip = state.data_ptr(), positions.data_ptr(), slot_ids.data_ptr()
+    out = torch.empty((T, D), dtype=out_dtype, device=x.device) if out_dtype is not None else None
+    if T:
+        _check(_fn("post_norm", "bn_post_norm")(
+            _code(kind), x.data_ptr(), y.data_ptr(), y.shape[0] if parts else 1, int(parts),
+            gain.data_ptr() if gain is not None else None, float(alpha), weight.data_ptr(), float(eps),
+            out.data_ptr() if out is not None else None, T, D, mu.data_ptr() if mu is not None else None, sp, stride, pp, ip,
+            _stream()), "post_norm")
+    return out
+
+
+def sigmoid_gate_(y: torch.Tensor, gate: torch.Tensor) -> None:
+    """In place: y [T, N] times sigmoid(gate) element by element (gate [T, N] may be columns of a wider tensor)."""
+    require_gpu()
+    _dev(y, "y", dims=2)
+    _dev(gate, "gate", y.dtype, 2)
+    if y.shape != gate.shape:
+        raise KernelError(f"sigmoid_gate_: y {tuple(y.shape)} and gate {tuple(gate.shape)} differ")
+    if y.numel():
+        _check(_fn("latent", "bn_sigmoid_gate")(_code(y.dtype), y.data_ptr(), _rows(y, "y"), gate.data_ptr(), _rows(gate, "gate"), 1,
+                                                y.shape[0], y.shape[1], _stream()), "sigmoid_gate")
+
+
 def rmsnorm_mean(a: torch.Tensor, wa: torch.Tensor, b: Optional[torch.Tensor], wb: Optional[torch.Tensor],
                  eps: float) -> torch.Tensor:
     """The mean of two branches [T, D], each under an RMSNorm of its own (float32 weights [D]); b None: a alone."""
@@ -1685,27 +1789,38 @@ def _state_rows(state: torch.Tensor, need: int, what: str) -> int:
     return state.stride(0)
 
 
-def token_shift(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, positions, seq_index, slot_ids) -> torch.Tensor:
+def token_shift(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, positions, seq_index, slot_ids, *, out_dtype=None,
+                seq_lens=None) -> torch.Tensor:
     """[n_mix, T, D]: h[t] + (h[t-1] - h[t]) * mu[s] for every mix s; the token before a step's first is read from the
     first D values of the sequence's state row (state: [slots, >= D], a view that starts at those values), and is 0 at
-    position 0.  Reads the state only."""
+    position 0.  out_dtype: the mixes' type (default: h's; h float32 may give bfloat16 mixes).  seq_lens None: reads the
+    state only (whoever uses the mixes stores the step's last h); seq_lens [sequences], the lengths behind the step: the
+    last row of every sequence replaces those D values."""
     require_gpu()
     _dev(h, "h", dims=2)
     _dev(mu, "mu", torch.float32, 2)
     T, D = h.shape
+    out_dtype = out_dtype or h.dtype
     if not h.is_contiguous() or mu.shape[1] != D or not mu.is_contiguous():
         raise KernelError("token_shift: h contiguous [T, D], mu contiguous [n_mix, D]")
+    if out_dtype != h.dtype and h.dtype != torch.float32:
+        raise KernelError(f"token_shift: h in {h.dtype} gives mixes of its own type, not {out_dtype}")
     stride = _state_rows(state, D, "token_shift")
     for t, nm, n in ((positions, "positions", T), (seq_index, "seq_index", T)):
         _dev(t, nm, torch.int32, 1)
         if t.numel() != n or not t.is_contiguous():
             raise KernelError(f"token_shift: {nm} has one entry per row")
     _dev(slot_ids, "slot_ids", torch.int32, 1)
-    out = torch.empty((mu.shape[0], T, D), dtype=h.dtype, device=h.device)
+    if seq_lens is not None:
+        _dev(seq_lens, "seq_lens", torch.int32, 1)
+        if seq_lens.numel() != slot_ids.numel() or not seq_lens.is_contiguous():
+            raise KernelError("token_shift: seq_lens has one entry per sequence")
+    out = torch.empty((mu.shape[0], T, D), dtype=out_dtype, device=h.device)
     if T:
-        _check(_fn("state_mixers", "bn_token_shift")(_code(h.dtype), out.data_ptr(), h.data_ptr(), mu.data_ptr(), state.data_ptr(),
-                                                     stride, positions.data_ptr(), seq_index.data_ptr(),
-                                                     slot_ids.data_ptr(), T, D, mu.shape[0], _stream()), "token_shift")
+        _check(_fn("state_mixers", "bn_token_shift")(_code(h.dtype), _code(out_dtype), out.data_ptr(), h.data_ptr(), mu.data_ptr(),
+                                                     state.data_ptr(), stride, positions.data_ptr(), seq_index.data_ptr(),
+                                                     slot_ids.data_ptr(), seq_lens.data_ptr() if seq_lens is not None else None,
+                                                     T, D, mu.shape[0], _stream()), "token_shift")
     return out
 
 

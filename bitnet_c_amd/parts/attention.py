@@ -30,6 +30,14 @@ split-half or in neighbouring pairs, over the first rope_dims dimensions) and ta
                  projection (tensors q_conv [heads head_dim, taps], k_conv [kv heads head_dim, taps], no bias; the last
                  column meets the current token, zeros before a sequence's first token); with value_is_key the values are
                  the keys as they leave it.  A sequence's last taps - 1 projected rows are a state beside its pages.
+  bias "qk"      biases on the query and key projections alone (tensors bq [heads head_dim], bk [kv heads head_dim]), added by
+                 the kernel that norms and stores; with value_is_key the values have the key's
+  qk_norm_weight False: the per-head norms have no weights (no tensors q_norm, k_norm)
+  head_temp      every score of a head times a number of the head (tensor temp [heads])
+  distance_slopes  one number per head: slope[h] * (i - j) is taken off the score of query i and key j
+  keep_first     with a window: the first keep_first positions stay visible however far back they are, at their true distances
+  out_gate       the heads' outputs side by side times sigmoid(W_g h), element by element (tensor wg [heads v_head_dim,
+                 hidden], its rows stacked behind the other projections')
   value_is_key   there is no value projection: kv head g's value is its key projection as projected, before the key's norm
                  and rotation (the tensor wv does not exist; the value heads are as wide as the key heads)
 """
@@ -55,14 +63,18 @@ class Attention(Part):
                  position: PartSpec, window: int = 0, bias: bool = False, v_head_dim: int = 0,
                  qk_norm_eps: float | None = None, q_temp_coef: float = 0.0, q_temp_every: int = 0,
                  distance_bias: bool = False, sink=False, qk_norm_span: str = "head", value_is_key: bool = False,
-                 conv_taps: int = 0):
+                 conv_taps: int = 0, qk_norm_weight: bool = True, head_temp: bool = False, distance_slopes=None,
+                 keep_first: int = 0, out_gate: bool = False):
         if n_heads % n_kv_heads:
             raise ValueError(f"attention: {n_heads} heads are not a multiple of {n_kv_heads} kv heads")
         if head_dim % 2 or head_dim < 2 or head_dim > ops.MAX_HEAD_DIM:
             raise ValueError(f"attention: head_dim {head_dim} is not supported by the kernels "
                              f"(even, at most {ops.MAX_HEAD_DIM})")
         self.hidden, self.H, self.Hkv, self.hs = int(hidden), int(n_heads), int(n_kv_heads), int(head_dim)
-        self.scale, self.window, self.has_bias = float(scale), int(window), bool(bias)
+        if bias not in (False, True, "qk"):
+            raise ValueError(f"attention: bias {bias!r} is neither False, True nor 'qk'")
+        self.qk_bias = bias == "qk"
+        self.scale, self.window, self.has_bias = float(scale), int(window), bool(bias) and not self.qk_bias
         self.position = POSITION_ENCODINGS.build(position)
         self.qkv, self.o = Linear(), Linear()
         self.vd = int(v_head_dim) or self.hs
@@ -77,6 +89,17 @@ class Attention(Part):
         self.conv_taps = int(conv_taps)
         if self.conv_taps < 0 or self.conv_taps > ops.CONV_MAX_TAPS:
             raise ValueError(f"attention: conv_taps {conv_taps} (at most {ops.CONV_MAX_TAPS})")
+        self.qk_norm_weight, self.head_temp, self.out_gate = bool(qk_norm_weight), bool(head_temp), bool(out_gate)
+        if not self.qk_norm_weight and (self.qk_norm_eps is None or qk_norm_span != "head"):
+            raise ValueError("attention: a norm without weights is a norm over each head (qk_norm_eps)")
+        self.distance_slopes = tuple(float(v) for v in distance_slopes) if distance_slopes is not None else None
+        if self.distance_slopes is not None and (len(self.distance_slopes) != self.H or self.distance_bias):
+            raise ValueError(f"attention: one distance slope per head ({self.H}), and no other distance bias beside them")
+        self.keep_first = int(keep_first)
+        if self.keep_first < 0 or (self.keep_first and not self.window):
+            raise ValueError(f"attention: keep_first {keep_first} belongs to a window")
+        if self.qk_bias and self.conv_taps:
+            raise ValueError("attention: a convolution on the projections comes without their biases")
         if qk_norm_span not in ("head", "projection"):
             raise ValueError(f"attention: qk_norm_span {qk_norm_span!r} is neither 'head' nor 'projection'")
         self.norm_projection = qk_norm_span == "projection"
@@ -84,15 +107,17 @@ class Attention(Part):
             raise ValueError("attention: a norm over the whole projection needs qk_norm_eps")
         self.general = (self.vd != self.hs or self.qk_norm_eps is not None or self.q_temp_every > 0
                         or self.distance_bias or self.sink or getattr(self.position, "interleaved", False)
-                        or self.value_is_key or self.conv_taps > 0)
+                        or self.value_is_key or self.conv_taps > 0 or self.qk_bias or self.head_temp
+                        or self.distance_slopes is not None or self.keep_first > 0 or self.out_gate)
         if self.general:
             if self.vd % 2 or self.vd < 2 or self.vd > ops.MAX_HEAD_DIM:
                 raise ValueError(f"attention: v_head_dim {self.vd} is not supported by the kernels (even, at most {ops.MAX_HEAD_DIM})")
             if self.has_bias:
                 raise ValueError("attention: head norms, a query temperature, a distance bias, a sink, a rotation in neighbouring "
-                                 "pairs, values of another width or values that are the keys come without projection biases")
+                                 "pairs, values of another width, values that are the keys, kept first positions or an output gate "
+                                 "come without projection biases, or with those of queries and keys alone")
             self.takes_deferred_norm = self.gives_lazy_delta = False
-        self.q_norm = self.k_norm = self.dist_a = self.dist_b = self.sink_values = self.conv_w = None
+        self.q_norm = self.k_norm = self.dist_a = self.dist_b = self.sink_values = self.conv_w = self.qk_b = self.temp = None
 
     @property
     def q_dim(self):
@@ -107,7 +132,13 @@ class Attention(Part):
              "wv": ParamSpec((self.Hkv * self.vd, self.hidden)), "wo": ParamSpec((self.hidden, self.H * self.vd))}
         if self.value_is_key:
             del t["wv"]
-        if self.qk_norm_eps is not None:
+        if self.out_gate:
+            t["wg"] = ParamSpec((self.H * self.vd, self.hidden))
+        if self.qk_bias:
+            t.update({"bq": ParamSpec((self.q_dim,), "normal"), "bk": ParamSpec((self.kv_dim,), "normal")})
+        if self.head_temp:
+            t["temp"] = ParamSpec((self.H,), "ones")
+        if self.qk_norm_eps is not None and self.qk_norm_weight:
             nq, nk = (self.q_dim, self.kv_dim) if self.norm_projection else (self.hs, self.hs)
             t.update({"q_norm": ParamSpec((nq,), "ones"), "k_norm": ParamSpec((nk,), "ones")})
         if self.distance_bias:
@@ -123,7 +154,7 @@ class Attention(Part):
 
     def load(self, tensors, device, dtype):
         # stacked on the device: the host holds no copy beside the file's own bytes
-        stacked = ("wq", "wk") if self.value_is_key else ("wq", "wk", "wv")
+        stacked = (("wq", "wk") if self.value_is_key else ("wq", "wk", "wv")) + (("wg",) if self.out_gate else ())
         w = torch.cat([upload(tensors[n], device, dtype) for n in stacked], dim=0).contiguous()
         b = None
         if self.has_bias:
@@ -131,8 +162,16 @@ class Attention(Part):
         self.qkv.load(w, b, device, dtype)
         self.o.load(tensors["wo"], tensors.get("bo") if self.has_bias else None, device, dtype)
         self.position.prepare(device)
-        if self.qk_norm_eps is not None:
+        if self.qk_norm_eps is not None and self.qk_norm_weight:
             self.q_norm, self.k_norm = (upload(tensors[n], device, torch.float32) for n in ("q_norm", "k_norm"))
+        elif self.qk_norm_eps is not None:                # weights of one
+            self.q_norm = self.k_norm = torch.ones(self.hs, dtype=torch.float32, device=device)
+        if self.qk_bias:
+            self.qk_b = torch.cat([upload(tensors[n], device, torch.float32) for n in ("bq", "bk")]).contiguous()
+        if self.head_temp:
+            self.temp = upload(tensors["temp"], device, torch.float32)
+        if self.distance_slopes is not None:
+            self.dist_a = torch.tensor(self.distance_slopes, dtype=torch.float64).to(torch.float32).to(device)
         if self.distance_bias:
             self.dist_a, self.dist_b = (upload(tensors[n], device, torch.float32) for n in ("dist_a", "dist_b"))
         if self.sink_learned:
@@ -149,7 +188,8 @@ class Attention(Part):
             state = None
             if self.conv_taps > 1:        # the projected query and key rows of the last taps - 1 positions, float32
                 state = StateNeed(((self.conv_taps - 1) * (self.q_dim + self.kv_dim),), torch.float32, device_addressed=True)
-            return CacheNeed(kv=KVNeed(self.Hkv, self.hs, self.window, v_head_dim=self.vd, v_layout="transposed"), state=state)
+            return CacheNeed(kv=KVNeed(self.Hkv, self.hs, self.window, v_head_dim=self.vd, v_layout="transposed",
+                                       keep_first=self.keep_first), state=state)
         return CacheNeed(kv=KVNeed(self.Hkv, self.hs, self.window))
 
     def wants_deferred_norm(self, ctx, rows: int) -> bool:
@@ -162,14 +202,14 @@ class Attention(Part):
                     and ops.can_fuse_decode(self.qkv.weight.dtype, self.H, self.Hkv, self.hs))
 
     def _forward_general(self, h, ctx, kv):
-        """Projections; norms, rotation and temperature with the cache write (one kernel); attention with its window,
-        distance bias and sink (prompt steps on the matrix cores where the sizes allow, else the vector kernel); the
+        """Projections; biases, norms, rotation and temperature with the cache write (one kernel); attention with its window,
+        distance bias, sink and output gate (prompt steps on the matrix cores where the sizes allow, else the vector kernel); the
         output projection."""
         H, Hkv, hs, vd = self.H, self.Hkv, self.hs, self.vd
         if isinstance(h, ops.DeferredNorm):
             h = h.materialize()
-        width = H * hs + Hkv * (hs if self.value_is_key else hs + vd)
-        if kv.writes:
+        width = H * hs + Hkv * (hs if self.value_is_key else hs + vd) + (H * vd if self.out_gate else 0)
+        if kv.writes or self.out_gate:
             qkv = self.qkv(h)
         else:
             qkv = torch.empty((h.shape[0], width), dtype=h.dtype, device=h.device)
@@ -190,17 +230,19 @@ class Attention(Part):
                           rope_dims=self.position.rope_dims, rope_interleaved=getattr(self.position, "interleaved", False),
                           seq_index=ctx.seq_index if kv.writes else None, block_table=kv.block_table if kv.writes else None,
                           k_pages=kv.k_pages if kv.writes else None, v_pages=kv.v_pages if kv.writes else None,
-                          v_transposed=True, v_from_k=self.value_is_key)
+                          v_transposed=True, v_from_k=self.value_is_key, bias=self.qk_b, head_temp=self.temp)
         out = torch.empty((h.shape[0], H * vd), dtype=h.dtype, device=h.device)
-        bias = (self.dist_a, self.dist_b) if self.distance_bias else None
+        bias = (self.dist_a, self.dist_b) if self.dist_a is not None else None
+        gate = qkv[:, width - H * vd:] if self.out_gate else None
+        mask = dict(window=self.window, keep_first=self.keep_first)
         on_matrix_cores = (ops.attention_general_supported(h.dtype, hs, vd) and ops.GENERAL_PROMPT_ON_MATRIX_CORES
                            and width % 8 == 0 and qkv.data_ptr() % 16 == 0)
         if ctx.is_decode and on_matrix_cores:
             n_splits, chunk, follows = ops.general_decode_plan(ctx.n_rows, H, Hkv, kv.max_len, self.window)
             ops.attention_general_decode(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, ctx.seq_lens, H, Hkv, hs, vd, self.scale,
-                                         window=self.window, n_splits=n_splits, chunk=chunk,
+                                         n_splits=n_splits, chunk=chunk,
                                          max_len_dev=ctx.max_len_dev if follows and n_splits > 1 else None,
-                                         distance_bias=bias, sink=self._sink())
+                                         distance_bias=bias, sink=self._sink(), gate=gate, **mask)
         elif ctx.is_decode:
             if not self.window:
                 n_splits, chunk = ops.decode_splits(ctx.n_rows, H, Hkv, kv.max_len, h.dtype, target_wgs=ops.VECTOR_DECODE_TARGET_WGS)
@@ -211,19 +253,21 @@ class Attention(Part):
                                                     target_wgs=ops.VECTOR_DECODE_TARGET_WGS)
             else:
                 n_splits, chunk = 1, 0                    # a short window is not split; a float32 cache sums in runs from position 0
-            ops.attention(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, H, Hkv, hs, self.scale, window=self.window,
+            ops.attention(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, H, Hkv, hs, self.scale,
                           seq_lens=ctx.seq_lens, n_splits=n_splits, chunk=chunk,
                           max_len_dev=ctx.max_len_dev if n_splits > 1 and not self.window else None, v_transposed=True, blocked=False,
-                          v_dim=vd, distance_bias=bias, sink=self._sink())
+                          v_dim=vd, distance_bias=bias, sink=self._sink(), **mask)
         elif on_matrix_cores:
             ops.attention_general_prompt(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, H, Hkv, hs, vd, self.scale,
                                          ctx.tiles(ops.GENERAL_PROMPT_TILE), distance_bias=bias, sink=self._sink(),
-                                         window=self.window)
+                                         gate=gate, **mask)
         else:
             _, _, qt = ops.attention_row_shape(H, Hkv, False)
-            ops.attention(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, H, Hkv, hs, self.scale, window=self.window,
+            ops.attention(qkv, out, kv.k_pages, kv.v_pages, kv.block_table, H, Hkv, hs, self.scale,
                           tiles=ctx.tiles(qt), qt=qt, v_transposed=True, blocked=False, v_dim=vd, distance_bias=bias,
-                          sink=self._sink())
+                          sink=self._sink(), **mask)
+        if gate is not None and not on_matrix_cores:      # the matrix-core kernels multiply by it as they store
+            ops.sigmoid_gate_(out, gate)
         return self.o(out)
 
     def _sink(self):

@@ -71,20 +71,24 @@ class KVNeed:
     the keys and the values inside a (page, kv head) as this library's matrix-core attention kernels load them
     (ops.blocked_page_index); nothing else reads such pages.  v_layout None asks for the layout
     that this library's attention kernels read at the cache's type and head size (ops.kernel_v_layout); a mixer with
-    kernels or torch code of its own names the layout it wants ("rows" or "transposed")."""
+    kernels or torch code of its own names the layout it wants ("rows" or "transposed").  keep_first (with a window): the
+    first keep_first positions of a sequence are kept however far back they are."""
     n_kv_heads: int
     head_dim: int
     window: int = 0
     v_head_dim: int = 0
     v_layout: Optional[str] = None
+    keep_first: int = 0
 
     V_LAYOUTS = ("rows", "transposed", "blocked")
 
     def __post_init__(self):
         if self.v_layout is not None and self.v_layout not in self.V_LAYOUTS:
             raise ValueError(f"KVNeed: v_layout {self.v_layout!r} is not one of {self.V_LAYOUTS}")
-        if self.n_kv_heads < 1 or self.head_dim < 1 or self.v_head_dim < 0 or self.window < 0:
+        if self.n_kv_heads < 1 or self.head_dim < 1 or self.v_head_dim < 0 or self.window < 0 or self.keep_first < 0:
             raise ValueError(f"KVNeed: sizes must be positive, got {self}")
+        if self.keep_first and not self.window:
+            raise ValueError(f"KVNeed: first positions are kept beside a window, got {self}")
         if self.v_layout == "blocked" and (self.head_dim % 32 or self.v_head_dim not in (0, self.head_dim)):
             raise ValueError(f"KVNeed: blocked pages need values as wide as keys and a head size that is a multiple of 32, got {self}")
 
@@ -197,6 +201,18 @@ class NormedDelta:
         self.delta, self.norm = delta, norm
 
 
+class PostNormedDelta:
+    """A part's output in a block whose norms stand behind the sums: the stream becomes norm(alpha * x + gain * delta).
+    `delta` [T, D] in the activations' type, or ops.PartialSums; gain [D] float32 or None (1); all in float32."""
+
+    def __init__(self, delta, norm, alpha: float, gain=None):
+        self.delta, self.norm, self.alpha, self.gain = delta, norm, float(alpha), gain
+
+    def apply(self, x: torch.Tensor, **rows):
+        from .. import ops
+        return ops.post_norm(x, self.delta, self.gain, self.alpha, self.norm.weight, self.norm.eps, **rows)
+
+
 class ResidualStream:
     """The float32 residual stream of a step.  A part's output is held back as `pending` and
     is added by the kernel of the next norm, so the sum is formed once, in float32, without a
@@ -214,7 +230,7 @@ class ResidualStream:
         self.pending = delta
 
     def _pending_tensor(self):
-        if isinstance(self.pending, NormedDelta):
+        if isinstance(self.pending, (NormedDelta, PostNormedDelta)):
             raise TypeError("an output with a norm of its own is added by flush() or normed()")
         if isinstance(self.pending, LazyDelta):
             self.pending = self.pending.compute()
@@ -225,11 +241,27 @@ class ResidualStream:
             from .. import ops
             p, self.pending = self.pending, None
             ops.add_normed_rmsnorm(self.x, p.delta, p.norm.weight, p.norm.eps)
+        if isinstance(self.pending, PostNormedDelta):
+            p, self.pending = self.pending, None
+            p.apply(self.x)
         if self.pending is not None:
             from .. import ops
             ops.residual_add(self.x, self._pending_tensor())
             self.pending = None
         return self.x
+
+    def mixed_with_previous(self, mu: torch.Tensor, state: torch.Tensor, ctx) -> torch.Tensor:
+        """x + (x' - x) * mu in the activations' type, x' the previous token's row of the stream as it stands here (zeros in
+        front of a sequence's first).  The last row of every sequence is kept in `state` (rows by slot, float32, at least as
+        wide as the stream).  In a decode step a held-back output that is normed with the sum is folded into the same
+        kernel."""
+        from .. import ops
+        if ctx.is_decode and isinstance(self.pending, PostNormedDelta):
+            p, self.pending = self.pending, None
+            return p.apply(self.x, out_dtype=ctx.act_dtype, mu=mu, state=state, positions=ctx.positions, slot_ids=ctx.slot_ids)
+        self.flush()
+        return ops.token_shift(self.x, mu.reshape(1, -1), state, ctx.positions, ctx.seq_index, ctx.slot_ids,
+                               out_dtype=ctx.act_dtype, seq_lens=ctx.seq_lens)[0]
 
     def normed(self, norm, out_dtype, rows=None, consumer=None, ctx=None):
         """The normed stream for the next part.  `consumer`: the part that will read it; when it
@@ -237,6 +269,11 @@ class ResidualStream:
         folded around, the result is an ops.DeferredNorm instead of a tensor.  With more rows than the fused
         products take, a consumer that has a method wants_deferred_norm(ctx, rows) is asked first (ctx: the step's
         context): one that would only apply the norm the plain way gets the plain norm, in one kernel instead of two."""
+        if isinstance(self.pending, PostNormedDelta):
+            if rows is None and getattr(norm, "passes_rows", False):
+                p, self.pending = self.pending, None
+                return p.apply(self.x, out_dtype=out_dtype)          # the sum, its norm and the new rows in one kernel
+            self.flush()
         if isinstance(self.pending, NormedDelta):
             # the held-back output's norm, the sum and this norm in one kernel; with a choice of rows the sum comes first
             if rows is None and getattr(norm, "normed_delta", False):

@@ -260,10 +260,32 @@ def _mutirax_configs(z):
     return (mut,) + _fazopel_configs(z)
 
 
+def _pafutar_configs(z):
+    """(Pafutar config.json, Fazopel config.json, Sonodra config.json, Llama config.json) of equal width, layers, attention
+    heads and dense feed-forwards: Pafutar with the window and 16 kept first tokens; Fazopel with its attention (causal over
+    every key) and the same feed-forward in every layer; Sonodra with its windowed attention of the same window and a gated
+    feed-forward of as many weights."""
+    att = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5)
+    dense, rot = dict(kind="dense", ff=z["ff"]), dict(base=500000.0, dims=z["rot_dims"])
+    gated = dict(kind="dense", ff=_llama_config(z)["intermediate_size"])
+
+    def layers(mixer, mlp):
+        return [dict(type="attention", mixer=mixer, mlp=mlp)] * z["layers"]
+    paf = dict(architecture="Pafutar", vocab=z["vocab"], width=z["width"], max_positions=8192, norm=dict(eps=1e-6),
+               embedding=dict(scale=8.0), postln_alpha=1.5,
+               layers=layers(dict(att, mask=dict(size=z["window"], keep_first=16)), dense))
+    faz = dict(architecture="Fazopel", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6), layers=layers(dict(att, rot=rot), dense))
+    son = dict(architecture="Sonodra", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6),
+               layers=layers(dict(att, mask=dict(size=z["window"]), rot=dict(base=10000.0, dims=z["rot_dims"])), gated))
+    return paf, faz, son, _llama_config(z)
+
+
 def _design_configs(design, z):
     """name -> config.json: the design, then what it is measured beside (the Llama-style decoder of equal width, layers,
     attention heads and (nearly) equal weight bytes read per token; for Fazopel also Sonodra, the closest of the others;
-    for Mutirax Fazopel and Sonodra)."""
+    for Mutirax Fazopel and Sonodra; for Pafutar both, with its own kind of layer in every layer)."""
+    if design == "pafutar":
+        return dict(zip(("pafutar", "fazopel", "sonodra", "llama"), _pafutar_configs(z)))
     if design == "mutirax":
         return dict(zip(("mutirax", "fazopel", "sonodra", "llama"), _mutirax_configs(z)))
     if design == "fazopel":
@@ -379,7 +401,7 @@ def main() -> int:
     ap.add_argument("--prompt-lens", default=None, metavar="LO,HI", help="prompt lengths of the decode batches")
     ap.add_argument("--prefill-tokens", type=int, default=PREFILL_TOKENS, help="tokens of the measured prompt step")
     ap.add_argument("--design-alone", action="store_true", help="with --design: the design alone, for profiling")
-    ap.add_argument("--design", choices=["sunusun", "sonodra", "fazopel", "mutirax"], default=None,
+    ap.add_argument("--design", choices=["sunusun", "sonodra", "fazopel", "mutirax", "pafutar"], default=None,
                     help="instead of the benchmark: prefill and decode of this design beside the Llama-style decoder of equal "
                          "width, heads, layers and weight bytes, at the sizes of --design-size (random weights; one JSON line)")
     ap.add_argument("--design-size", choices=sorted(DESIGN_SIZES), default="2048")

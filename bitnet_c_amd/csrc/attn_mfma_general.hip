@@ -57,9 +57,20 @@ __device__ __forceinline__ bf16x8 ag_ld16(const bf16* p) {
     return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p));
 }
 
-// the score's distance bias in the exponent's base 2; a ln(x) log2(e) = a log2(x)
-__device__ __forceinline__ float ag_bias2(float a, float b, bool linear, float dist) {
-    return linear ? a * AG_LOG2E * dist : a * __log2f(1.0f + b * dist);
+// a lane's eight scores (keys first .. first + 7) of the query at qpos: scaled, less the distance bias, in the exponent's
+// base 2.  bias: 0 none, 1 logarithmic (a ln(1 + b d) log2(e) = a log2(1 + b d)), 2 linear (a d, with log2(e) in a)
+__device__ __forceinline__ void ag_scores(float (&s)[8], const f32x4& s0, const f32x4& s1, float scale2, int bias, float ba, float bb,
+                                          int qpos, int first) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s[e] = (e < 4 ? s0[e & 3] : s1[e & 3]) * scale2;
+    const float dist = (float)(qpos - first);
+    if (bias == 2) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s[e] = fmaf(-ba, dist - (float)e, s[e]);
+    } else if (bias == 1) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s[e] -= ba * __log2f(1.0f + bb * (dist - (float)e));
+    }
 }
 
 // four consecutive outputs of a head and, with a gate, times the sigmoids of the four gate values beside them:
@@ -98,8 +109,8 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
         for (int c = 0; c < DC; ++c) qf[c] = ag_ld16(qp + 32 * c);
     }
     const float scale2 = a.scale * AG_LOG2E;
-    const bool linear = a.dist_b == nullptr;
-    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a && !linear ? a.dist_b[head] : 0.f;
+    const int bias = a.dist_a ? (a.dist_b ? 1 : 2) : 0;
+    const float ba = bias ? a.dist_a[head] * (bias == 2 ? AG_LOG2E : 1.0f) : 0.f, bb = bias == 1 ? a.dist_b[head] : 0.f;
     f32x4 acc[DT];
 #pragma unroll
     for (int t = 0; t < DT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -143,12 +154,12 @@ __global__ __launch_bounds__(AG_WAVES * BN_WAVE) void attn_general_prompt_kernel
         for (int t = 0; t < DT; ++t) va[t] = ag_ld16(vbase + (size_t)t * 16 * BN_PAGE);
         // this lane's eight scores: keys kb + 8 g + e, e = 4 h + r
         float s[8];
+        ag_scores(s, st0, st1, scale2, bias, ba, bb, qpos, kb + 8 * g);
         float mx = -INFINITY;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int key = kb + 8 * g + e;
-            float v = (e < 4 ? st0[e & 3] : st1[e & 3]) * scale2;
-            if (a.dist_a) v -= ag_bias2(ba, bb, linear, (float)(qpos - key));
+            float v = s[e];
             if (!col_ok || key > qpos || key >= k_hi || (key <= q_lo && key >= keep)) v = -INFINITY;
             s[e] = v;
             mx = fmaxf(mx, v);
@@ -275,8 +286,8 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
         for (int c = 0; c < DC; ++c) qf[c] = ag_ld16(qp + 32 * c);
     }
     const float scale2 = a.scale * AG_LOG2E;
-    const bool linear = a.dist_b == nullptr;
-    const float ba = a.dist_a ? a.dist_a[head] : 0.f, bb = a.dist_a && !linear ? a.dist_b[head] : 0.f;
+    const int bias = a.dist_a ? (a.dist_b ? 1 : 2) : 0;
+    const float ba = bias ? a.dist_a[head] * (bias == 2 ? AG_LOG2E : 1.0f) : 0.f, bb = bias == 1 ? a.dist_b[head] : 0.f;
     f32x4 acc[DT];
 #pragma unroll
     for (int t = 0; t < DT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -310,12 +321,12 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
 #pragma unroll
         for (int t = 0; t < DT; ++t) va[t] = ag_ld16(vbase + (size_t)t * 16 * BN_PAGE);
         float s[8];
+        ag_scores(s, st0, st1, scale2, bias, ba, bb, qpos, kb + 8 * g);
         float mx = -INFINITY;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int key = kb + 8 * g + e;
-            float v = (e < 4 ? st0[e & 3] : st1[e & 3]) * scale2;
-            if (a.dist_a) v -= ag_bias2(ba, bb, linear, (float)(qpos - key));
+            float v = s[e];
             if (!col_ok || (key < k_lo && key >= keep) || key >= k_hi) v = -INFINITY;
             s[e] = v;
             mx = fmaxf(mx, v);

@@ -11,6 +11,7 @@
 // DUAL: W holds two row blocks (gate rows n, up rows up_off + n); the epilogue writes
 // act(gate) * up, act one of the kinds of bn_gate_act (silu(g) = g / (1 + exp(-g)) for this
 // architecture, src/transformer/cpu_backend.c:385-391).
+// Neither: Y is the product, or with act BN_ACT_RELU2 the square of its positive part.
 // GLU8: the same product with gate and up rows interleaved in blocks of 8 (rows 16t..16t+7 are
 // gate rows 8t..8t+7, rows 16t+8..16t+15 the up rows of the same columns): every 16-row tile holds
 // both halves of 8 result columns, so the plain kernel does it with half the loads in flight.
@@ -143,7 +144,8 @@ __global__ __launch_bounds__((DUAL && MT >= 3) ? 512 : 1024) void skinny_gemm_ke
             if ((l & 8) == 0 && m < M && nn < N)
                 Y[(size_t)m * ldy + (n0 >> 1) + (l & 7)] = from_f32<TO>(bn_gate_act(v, act) * up);
         } else if (m < M && nn < N) {
-            const float y = DUAL ? bn_gate_act(v, act) * u : v;
+            const float p = fmaxf(v, 0.f);
+            const float y = DUAL ? bn_gate_act(v, act) * u : (act == BN_ACT_RELU2 ? p * p : v);
             Y[(size_t)m * ldy + nn] = from_f32<TO>(y);
         }
     }
@@ -453,7 +455,8 @@ extern "C" int bn_skinny_gemm_supports(int M, int N, int K, int ldx, int ldw) {
 // out_dtype: type of Y (bf16 or float32).  dual == 1: N is the width of the result and W has
 // the gate rows at [0, N) and the up rows at [up_off, up_off + N).  dual == 2: W has 2N rows, gate
 // and up interleaved in blocks of 8 (N a multiple of 8); the result has N columns.  act: the gate's activation
-// (BN_ACT_*), used when dual != 0.
+// (BN_ACT_*) when dual != 0; with dual == 0 BN_ACT_RELU2 squares the positive part of every result (a feed-forward without
+// a gate) and any other value leaves the product as it is.
 // tile_rows > 0: W is the streamed copy (common.h) with that many rows a tile and ldw its tiles along K; up to 16 rows,
 // dual == 0.
 extern "C" int bn_skinny_gemm(int out_dtype, const void* X, const void* W, void* Y, int M, int N, int K,

@@ -609,6 +609,25 @@ def linear(x: torch.Tensor, w: torch.Tensor, out_dtype=None, *, allow_library: O
     return _tiled(x, w, out_dtype)
 
 
+def linear_unary(x: torch.Tensor, w: torch.Tensor, activation: str, streamed: Optional[StreamedWeight] = None) -> torch.Tensor:
+    """activation(linear(x, w)) (one of UNARY_ACTIVATIONS): a feed-forward's first product without a gate.  bf16 steps of up
+    to 16 rows form relu2 in the product's own kernel; everything else is the product, then the activation's kernel."""
+    require_gpu()
+    _dev(x, "x", dims=2)
+    _dev(w, "w", x.dtype, 2)
+    M, K = x.shape
+    N = w.shape[0]
+    if (activation == "relu2" and x.dtype == torch.bfloat16 and 1 <= M <= SKINNY_ROWS and w.shape[1] == K
+            and (x.data_ptr() | w.data_ptr()) % 16 == 0 and skinny_supported(M, N, K, _rows(x, "x"), _rows(w, "w"))):
+        y = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
+        wp, wl, tiled = _weight_arg(w, streamed, "linear_unary")
+        _check(_fn("skinny_gemm", "bn_skinny_gemm")(_code(torch.bfloat16), x.data_ptr(), wp, y.data_ptr(), M, N, K, _rows(x, "x"),
+                                                    wl, N, 0, 0, _act("relu2"), tiled, _stream()), "skinny_gemm(relu2)")
+        return y
+    y = linear(x, w, streamed=streamed)
+    return unary_act(y, activation, out=y)
+
+
 def interleave_gate_up(w_gate: torch.Tensor, w_up: torch.Tensor) -> torch.Tensor:
     """[2F, K] with gate and up rows alternating in blocks of 8 (F a multiple of 8): rows
     16t..16t+7 are gate rows 8t..8t+7, rows 16t+8..16t+15 the up rows of the same columns.  A

@@ -116,7 +116,7 @@ class Attention(Part):
                 raise ValueError("attention: head norms, a query temperature, a distance bias, a sink, a rotation in neighbouring "
                                  "pairs, values of another width, values that are the keys, kept first positions or an output gate "
                                  "come without projection biases, or with those of queries and keys alone")
-            self.takes_deferred_norm = self.gives_lazy_delta = False
+            self.takes_deferred_norm = False
         self.q_norm = self.k_norm = self.dist_a = self.dist_b = self.sink_values = self.conv_w = self.qk_b = self.temp = None
 
     @property
@@ -201,7 +201,7 @@ class Attention(Part):
         return bool(ctx.is_decode and fuse_ok and inv_freq is not None and not self.has_bias and ops.LIBRARY_PRODUCTS
                     and ops.can_fuse_decode(self.qkv.weight.dtype, self.H, self.Hkv, self.hs))
 
-    def _forward_general(self, h, ctx, kv):
+    def _forward_general(self, h, ctx, kv, lazy_ok: bool = False):
         """Projections; biases, norms, rotation and temperature with the cache write (one kernel); attention with its window,
         distance bias, sink and output gate (prompt steps on the matrix cores where the sizes allow, else the vector kernel); the
         output projection."""
@@ -268,7 +268,7 @@ class Attention(Part):
                           sink=self._sink(), **mask)
         if gate is not None and not on_matrix_cores:      # the matrix-core kernels multiply by it as they store
             ops.sigmoid_gate_(out, gate)
-        return self.o(out)
+        return self.o.lazy(out) if lazy_ok else self.o(out)
 
     def _sink(self):
         return self.sink_values if self.sink_learned else self.sink
@@ -281,7 +281,7 @@ class Attention(Part):
 
     def forward(self, h, ctx, kv, lazy_ok: bool = False):
         if self.general:
-            return self._forward_general(h, ctx, kv)
+            return self._forward_general(h, ctx, kv, lazy_ok)
         H, Hkv, hs = self.H, self.Hkv, self.hs
         last = self.o.lazy if lazy_ok else self.o
         fuse_ok, inv_freq = self.position.fusable(hs)

@@ -39,8 +39,11 @@ class DenseFFN(Part):
         return [self.up, self.down]
 
     def forward(self, h, ctx, lazy_ok: bool = False):
-        a = self.up(h)
-        ops.unary_act(a, self.activation, out=a)
+        if isinstance(h, ops.DeferredNorm):
+            a = self.up(h)
+            ops.unary_act(a, self.activation, out=a)
+        else:
+            a = ops.linear_unary(h, self.up.weight, self.activation, self.up.streamed)
         return self.down.lazy(a) if lazy_ok else self.down(a)
 
 

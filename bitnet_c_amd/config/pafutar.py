@@ -10,8 +10,8 @@ The mixer is "attention" (parts/attention.py): grouped-query attention without a
 projections themselves; biases on the query and key projections; an RMSNorm without weights over every query and key head;
 scores times a number per head, less slope_h times the distance, slope_h = 2^(-8 (h + 1) / heads); a sliding window beside
 which a sequence's first tokens stay visible; the heads' outputs times sigmoid(W_g h).  The feed-forward is "dense" (squared
-relu, no gate); "mlp": null leaves the second half out.  A layer with "weights_of": j has no tensors of its own: it runs
-layer j's weights with pages and a state of its own, which the plan's schedule says by naming layer j twice.
+relu, no gate); "mlp": null leaves the second half out.  "weights_of": j runs layer j's block once more, norms and vectors
+included, over other pages and another state row: the plan's schedule names that block twice.
 
 config.json keys: architecture, vocab, width, max_positions, norm.eps, embedding.scale, postln_alpha,
   layers[] = {type: "attention", mixer, mlp, weights_of?} with

@@ -72,13 +72,31 @@ def visible(i: int, mask) -> list:
     return [j for j in range(i + 1) if i - j < size or j < kept]
 
 
+def attend(q, k, v, pos0: int, mask, scale: float, temp, slopes) -> torch.Tensor:
+    """q [T, H, d] of the positions pos0 .. pos0 + T - 1 over k, v [P, G, *] of the positions 0 .. P - 1: the score of query
+    i and key j is (q . k) * scale * temp[head] - slope[head] * (i - j), the softmax runs over the keys that the mask
+    leaves.  Returns [T, H, width of v]."""
+    T, H = q.shape[:2]
+    G = k.shape[1]
+    out = torch.zeros((T, H, v.shape[-1]), dtype=F64)
+    for t in range(T):
+        i = pos0 + t
+        js = torch.tensor(visible(i, mask))
+        far = (i - js).to(F64)
+        for hd in range(H):
+            g = hd // (H // G)
+            s = (k[js, g] @ q[t, hd]) * scale * temp[hd] - slopes[hd] * far
+            e = torch.exp(s - s.max())
+            out[t, hd] = (e / e.sum()) @ v[js, g]
+    return out
+
+
 def windowed_attention(h, W, p, m, eps, pos0: int = 0, past=None, round_to=None):
     """Grouped-query attention whose values are its key projections (bias included, before the key's norm).  Every query
-    and key head is divided by its own root mean square, no weight; the score of query i and key j is
-    (q . k) * scale * temp[head] - slope[head] * (i - j), the softmax runs over the keys that the mask leaves; the heads'
-    outputs side by side are multiplied by sigmoid(W_g h); then W_o.  past: (keys [P, G, d], values [P, G, d]) of earlier
-    positions.  Returns (output [T, D], (keys, values) of all positions so far).  round_to: queries, keys, values and the
-    gated outputs are rounded to this type where an engine of that type stores them."""
+    and key head is divided by its own root mean square, no weight; attend(); the heads' outputs side by side are multiplied
+    by sigmoid(W_g h); then W_o.  past: (keys [P, G, d], values [P, G, d]) of earlier positions.  Returns (output [T, D],
+    (keys, values) of all positions so far).  round_to: queries, keys, values and the gated outputs are rounded to this type
+    where an engine of that type stores them."""
     rd = (lambda t: t.to(round_to).to(F64)) if round_to is not None else (lambda t: t)
     T = h.shape[0]
     H, G, d = m["heads"], m.get("kv_heads", m["heads"]), m["dim"]
@@ -88,16 +106,7 @@ def windowed_attention(h, W, p, m, eps, pos0: int = 0, past=None, round_to=None)
     q = rd(unit_rms(q, eps))
     if past is not None:
         k, v = torch.cat([past[0], k]), torch.cat([past[1], v])
-    out = torch.zeros((T, H, d), dtype=F64)
-    for t in range(T):
-        i = pos0 + t
-        js = torch.tensor(visible(i, m.get("mask")))
-        far = (i - js).to(F64)
-        for hd in range(H):
-            g = hd // (H // G)
-            s = (k[js, g] @ q[t, hd]) * m["scale"] * W[p + "temp"][hd] - head_slope(hd, H) * far
-            e = torch.exp(s - s.max())
-            out[t, hd] = (e / e.sum()) @ v[js, g]
+    out = attend(q, k, v, pos0, m.get("mask"), m["scale"], W[p + "temp"], [head_slope(hd, H) for hd in range(H)])
     y = rd(out.reshape(T, H * d) * sigmoid(h @ W[p + "g"].T))
     return y @ W[p + "o"].T, (k, v)
 

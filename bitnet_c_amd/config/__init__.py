@@ -1,4 +1,4 @@
-"""Typed configurations and the architecture registry; importing registers "llama", "Sunusun", "Sonodra", "Fazopel", "Mutirax" and "Pafutar"."""
+"""Typed configurations and the architecture registry; importing registers "llama", "Sunusun", "Sonodra", "Fazopel", "Mutirax", "Pafutar" and "Zenasun"."""
 from .base import (Architecture, ConfigError, architecture_for, architecture_names, load_config,
                    read_config_json, register_architecture)
 from .llama import LlamaConfig, RopeScaling
@@ -7,4 +7,5 @@ from .sonodra import SonodraConfig
 from .fazopel import FazopelConfig
 from .mutirax import MutiraxConfig
 from .pafutar import PafutarConfig
+from .zenasun import ZenasunConfig
 from . import llama_plan  # noqa: F401  (registration)

@@ -427,10 +427,14 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_combine_kernel(bf16* __r
     }
 }
 
-static bool ag_size(int x, int unit) { return x == unit || x == 2 * unit || x == 3 * unit || x == 4 * unit || x == 8 * unit; }
+static bool ag_size(int x) { return x == 32 || x == 64 || x == 96 || x == 128 || x == 192 || x == 256; }
 
-// 1 if the kernels take these head sizes (keys 32, 64, 96, 128 or 256 wide, values 32, 64, 96, 128, 192 or 256)
-extern "C" int bn_attn_general_supports(int hs, int vd) { return (ag_size(hs, 32) && (ag_size(vd, 32) || vd == 192)) ? 1 : 0; }
+// 1 if the kernels take these head sizes (keys 32, 64, 96, 128, 160, 192 or 256 wide, values from the same list without 160;
+// keys 160 or 192 wide are a latent beside a rotated part: values at least 64 wide)
+extern "C" int bn_attn_general_supports(int hs, int vd) {
+    if (hs == 160 || hs == 192) return ag_size(vd) && vd >= 64 && vd <= hs ? 1 : 0;
+    return ag_size(hs) && ag_size(vd) ? 1 : 0;
+}
 
 template <int DC>
 static int ag_launch_dt(const GenArgs& a, int vd, dim3 grid, hipStream_t s) {
@@ -469,6 +473,8 @@ extern "C" int bn_attn_general_prompt(const void* q, int q_stride, void* out, in
         case 2: return ag_launch_dt<2>(a, vd, grid, s);
         case 3: return ag_launch_dt<3>(a, vd, grid, s);
         case 4: return ag_launch_dt<4>(a, vd, grid, s);
+        case 5: return ag_launch_dt<5>(a, vd, grid, s);
+        case 6: return ag_launch_dt<6>(a, vd, grid, s);
         case 8: return ag_launch_dt<8>(a, vd, grid, s);
     }
     return BN_ERR_ARG;
@@ -519,6 +525,8 @@ extern "C" int bn_attn_general_decode(const void* q, int q_stride, void* out, in
         case 2: rc = ag_launch_decode_dt<2>(a, vd, grid, s); break;
         case 3: rc = ag_launch_decode_dt<3>(a, vd, grid, s); break;
         case 4: rc = ag_launch_decode_dt<4>(a, vd, grid, s); break;
+        case 5: rc = ag_launch_decode_dt<5>(a, vd, grid, s); break;
+        case 6: rc = ag_launch_decode_dt<6>(a, vd, grid, s); break;
         case 8: rc = ag_launch_decode_dt<8>(a, vd, grid, s); break;
     }
     if (rc != 0 || n_splits == 1) return rc;

@@ -1,4 +1,5 @@
-// Attention over the paged cache for any even head size up to 256, any number of heads and
+// Attention over the paged cache for any even head size up to 256 (keys up to 576 and values up to 512 wide where a latent
+// is the one head of the cache), any number of heads and
 // kv groups, float32 or bf16 cache, written on the vector ALUs.  Head sizes whose rows are
 // not whole 16-byte groups are staged element by element and padded with zeros in shared
 // memory to the next multiple of 8, which changes no sum.
@@ -476,6 +477,13 @@ static int launch_rows(const AttnArgs& a, int n_tiles, hipStream_t s) {
     const int G = a.H / a.Hkv;
     const int n_head_tiles = (G + a.GT - 1) / a.GT;
     const size_t smem = attn_smem_bytes(RT, a.hs, a.vd, a.KT, (int)sizeof(T));
+    static bool raised = false;              // rows wider than a head's: beyond the default limit of dynamic shared memory
+    if (smem > 64 * 1024 && !raised) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(attn_rows_kernel<T, RT>),
+                                                 hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        if (e != hipSuccess) return (int)e;
+        raised = true;
+    }
     hipLaunchKernelGGL((attn_rows_kernel<T, RT>), dim3(n_tiles, a.Hkv * n_head_tiles, a.n_splits),
                        dim3(ATT_THREADS), smem, s, a);
     return bn_launch_status();
@@ -494,7 +502,7 @@ static int launch_rows_rt(const AttnArgs& a, int RT, int n_tiles, hipStream_t s)
 }
 
 // Keys per tile: the largest of 64, 32, 16 whose shared memory stays within 64 KB for the widest
-// workgroup (16 rows); 0 if none does.  It is a function of the cache type and the head size alone,
+// workgroup (16 rows); 16 for rows so wide that none does and that fit into a CU's 160 KB; 0 beyond.  It is a function of the cache type and the head size alone,
 // never of the rows a launch happens to hold: a query's keys are then cut into the same tiles, and
 // its sums formed in the same order, whether it arrives alone, in a prompt or in a batch (the
 // reference keeps one order per kernel, src/transformer/gqa_scalar.c:61-121).
@@ -502,7 +510,7 @@ static int attn_key_tile(int dtype, int hs, int vd) {
     const int elt = dtype == BN_DT_F32 ? 4 : 2;
     for (int kt = 64; kt >= 16; kt >>= 1)
         if (attn_smem_bytes(16, hs, vd, kt, elt) <= 64 * 1024) return kt;
-    return 0;
+    return attn_smem_bytes(16, hs, vd, 16, elt) <= 160 * 1024 ? 16 : 0;
 }
 extern "C" int bn_attn_rows_key_tile(int dtype, int hs) { return attn_key_tile(dtype, hs, hs); }
 
@@ -517,11 +525,11 @@ extern "C" int bn_attn_rows(int dtype, const void* q, int q_stride, void* out, i
                             int v_transposed, const int* max_len, int fold, int vd, const float* dist_a,
                             const float* dist_b, int sink, const float* sink_values, int keep_first, hipStream_t s) {
     if (vd == 0) vd = hs;
-    if (vd < 2 || vd > BN_MAX_HEAD_DIM || vd % 2 || (dist_b && !dist_a)) return BN_ERR_ARG;
+    if (vd < 2 || vd > BN_MAX_LATENT_VALUE || vd % 2 || (dist_b && !dist_a)) return BN_ERR_ARG;
     if (n_tiles <= 0 || n_tokens <= 0 || H <= 0 || Hkv <= 0 || H % Hkv) return BN_ERR_ARG;
     // fold mode: runs of whole pages; a split is one run, and the runs' length does not follow the longest sequence
     if (fold < 0 || fold % BN_PAGE || (fold > 0 && n_splits > 1 && (chunk != fold || max_len))) return BN_ERR_ARG;
-    if (hs < 2 || hs > BN_MAX_HEAD_DIM || hs % 2) return BN_ERR_ARG;
+    if (hs < 2 || hs > BN_MAX_LATENT_KEY || hs % 2) return BN_ERR_ARG;
     if (GT <= 0 || GT > RT || (GT & (GT - 1)) || RT > 16 || (RT & (RT - 1))) return BN_ERR_ARG;
     if (n_splits < 1 || window < 0 || keep_first < 0) return BN_ERR_ARG;
     if (n_splits > 1 && (!part_o || !part_ml || (!max_len && (chunk <= 0 || chunk % BN_PAGE)))) return BN_ERR_ARG;

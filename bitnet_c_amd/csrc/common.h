@@ -15,6 +15,10 @@
 // every sum in the order in which a prompt step forms it, so that float32 logits do not depend on how a sequence was cut.
 #define BN_F32_FOLD_KEYS 2048
 #define BN_MAX_HEAD_DIM 256   // the attention kernels take every even head size up to this; the configuration reads this line too
+// A latent beside a rotated part is one wide "head" that all query heads share: the vector attention kernel takes key rows
+// up to this width, and values up to that one.
+#define BN_MAX_LATENT_KEY 576
+#define BN_MAX_LATENT_VALUE 512
 
 // The streamed copy of a bf16 weight matrix W[N, K], for the kernels that read W once per call in the operand layout of
 // v_mfma_f32_16x16x32_bf16 (lane l = r + 16 g holds columns 8 g .. 8 g + 7 of row r of a 16 x 32 block): tile (a, b) is rows

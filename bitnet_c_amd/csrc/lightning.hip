@@ -2,6 +2,8 @@
 //
 //     S_t = decay S_(t-1) + k_t v_t^T,      o_t = S_t^T q_t,      q, k, v = silu of their projections
 //
+// or, in the form of retention, q, k and v as projected, with the first rope_dims dimensions of every query and key head
+// rotated by the token's position (dimension i with i + rope_dims / 2, angle position * inv_freq[i]); k times a constant;
 // for prompt and decode steps alike.  The state lives in the cache's state area, [slot][head][dk][dv] float32; a kernel
 // finds a sequence's row through the step's device-side slot ids and its tokens either through a list of tiles (one tile
 // a sequence: sequence, first row, rows, position of the first; a tile of no rows is skipped) or, tiles == null, as row
@@ -17,7 +19,7 @@
 //                        This "chain" form serves decode steps, key widths above LC_MAX_DIM and prompt steps of so
 //                        many sequences that it fills the chip (bn_lightning_prefers_chunks).
 //   the chunked form     other prompt steps: a workgroup owns (sequence, head, 16 value columns) and takes the tokens in
-//                        chunks of 64, from a float32 copy of silu(q), silu(k), silu(v) that a kernel in front makes.  With d the decay, S the state before the chunk, n its tokens:
+//                        chunks of 64, from a float32 copy of the recurrence's q, k and v that a kernel in front makes.  With d the decay, S the state before the chunk, n its tokens:
 //                            A_ij = (q_i . k_j) d^(i-j) for j <= i,    o_i = sum_j A_ij v_j + d^(i+1) S^T q_i,
 //                            S   <- d^n S + sum_j d^(n-1-j) k_j v_j^T
 //                        which is the chain's sum in another order.  All four products run on the matrix cores in float32
@@ -49,6 +51,22 @@ __device__ __forceinline__ LaRange la_range(const int* tiles, const int* seq_len
 
 __device__ __forceinline__ float la_silu(float z) { return z / (1.0f + expf(-z)); }
 
+// what a projection passes on its way into the recurrence
+struct LaFeed {
+    int silu;                 // 1: q, k and v pass a silu; 0: as projected
+    int rope_dims;            // even; 0: no rotation (of q and k, behind the silu)
+    const float* inv_freq;    // [rope_dims / 2]
+    float k_scale;            // k times this, behind everything else
+};
+
+__device__ __forceinline__ float la_act(float z, int silu) { return silu ? la_silu(z) : z; }
+
+// the pair (u, v) turned by the angle whose sine and cosine are sn and cs
+__device__ __forceinline__ void la_turn(float& u, float& v, float sn, float cs) {
+    const float a = u * cs - v * sn, b = v * cs + u * sn;
+    u = a; v = b;
+}
+
 struct LaArgs {
     const void* x;            // [T, ld]: the projections side by side
     float* o;                 // [T, H dv] float32
@@ -59,6 +77,7 @@ struct LaArgs {
     const int* seq_lens;      // [B] when tiles is null
     const int* slot_ids;      // [sequences of the step]
     int ld, q_col, k_col, v_col, H, dk, dv;
+    LaFeed feed;
     const float* pq;          // the chunked form's copy of q, k and v (see lightning_prepare_kernel) and its sizes
     const float* pk;
     const float* pv;
@@ -87,21 +106,38 @@ __global__ __launch_bounds__(LA_THREADS) void lightning_scan_kernel(LaArgs a) {
     float* o = a.o + (size_t)sr.row0 * a.H * a.dv + (size_t)head * a.dv + c0;
     for (int t0 = 0; t0 < sr.n; t0 += LA_TC) {
         const int nt = min(LA_TC, sr.n - t0);
+        const int rd = a.feed.rope_dims, half = rd / 2;
         for (int idx = tid; idx < LA_TC * DKP; idx += LA_THREADS) {
             const int tt = idx / DKP, r = idx - tt * DKP;
+            if (r < rd) continue;                        // the rotated dimensions, pair by pair, below
             float qv = 0.f, kv = 0.f;
             if (tt < nt && r < a.dk) {
                 const T* row = x + (size_t)(t0 + tt) * a.ld + (size_t)head * a.dk + r;
-                qv = la_silu(to_f32(row[a.q_col]));
-                kv = la_silu(to_f32(row[a.k_col]));
+                qv = la_act(to_f32(row[a.q_col]), a.feed.silu);
+                kv = la_act(to_f32(row[a.k_col]), a.feed.silu) * a.feed.k_scale;
             }
             q_s[idx] = qv;
             k_s[idx] = kv;
         }
+        for (int idx = tid; idx < LA_TC * half; idx += LA_THREADS) {
+            const int tt = idx / half, r = idx - tt * half;
+            float q0 = 0.f, q1 = 0.f, k0 = 0.f, k1 = 0.f;
+            if (tt < nt) {
+                const T* row = x + (size_t)(t0 + tt) * a.ld + (size_t)head * a.dk + r;
+                float sn, cs;
+                sincosf((float)(sr.pos0 + t0 + tt) * a.feed.inv_freq[r], &sn, &cs);
+                q0 = la_act(to_f32(row[a.q_col]), a.feed.silu); q1 = la_act(to_f32(row[a.q_col + half]), a.feed.silu);
+                k0 = la_act(to_f32(row[a.k_col]), a.feed.silu); k1 = la_act(to_f32(row[a.k_col + half]), a.feed.silu);
+                la_turn(q0, q1, sn, cs);
+                la_turn(k0, k1, sn, cs);
+            }
+            q_s[tt * DKP + r] = q0; q_s[tt * DKP + half + r] = q1;
+            k_s[tt * DKP + r] = k0 * a.feed.k_scale; k_s[tt * DKP + half + r] = k1 * a.feed.k_scale;
+        }
         for (int idx = tid; idx < LA_TC * LA_CB; idx += LA_THREADS) {
             const int tt = idx / LA_CB, cc = idx - tt * LA_CB;
             v_s[idx] = (tt < nt && c0 + cc < a.dv)
-                           ? la_silu(to_f32(x[(size_t)(t0 + tt) * a.ld + a.v_col + (size_t)head * a.dv + c0 + cc])) : 0.f;
+                           ? la_act(to_f32(x[(size_t)(t0 + tt) * a.ld + a.v_col + (size_t)head * a.dv + c0 + cc]), a.feed.silu) : 0.f;
         }
         __syncthreads();
         for (int tt = 0; tt < nt; ++tt) {
@@ -145,23 +181,32 @@ __global__ __launch_bounds__(LA_THREADS) void lightning_scan_kernel(LaArgs a) {
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-// The chunked form reads a copy of the step's q, k and v that one kernel makes first: silu applied, float32, head by
+// The chunked form reads a copy of the step's q, k and v that one kernel makes first: silu and rotation applied, float32, head by
 // head ([H][T][dks] for q and for k, then [H][T][dvs] for v; dks and dvs the widths rounded up to a multiple of 4, the
 // elements behind a width zero).  A chunk of one head is then one run of consecutive bytes instead of 64 short pieces a
 // whole row of projections apart, every load is 16 bytes, and silu is taken once and not by every workgroup that shares
-// a head's q and k.
+// a head's q and k.  A row's sines and cosines are formed once and shared by all of its heads.
 struct LcPrepArgs {
     const void* x;            // [T, ld]
     float* q;                 // [H][T][dks]
     float* k;                 // [H][T][dks]
     float* v;                 // [H][T][dvs]
     int T, ld, q_col, k_col, v_col, H, dk, dv, dks, dvs;
+    LaFeed feed;
+    const int* positions;     // [T] with a rotation; < 0: a padding row (its copy is not read)
 };
 
 template <typename T>
 __global__ __launch_bounds__(256) void lightning_prepare_kernel(LcPrepArgs a) {
+    __shared__ float2 turn[LA_MAX_DIM / 2];              // (sine, cosine) of the row's angles
     const int t = blockIdx.x;
     const T* row = reinterpret_cast<const T*>(a.x) + (size_t)t * a.ld;
+    const int half = a.feed.rope_dims / 2;
+    if (half > 0) {
+        const float pos = (float)a.positions[t];
+        for (int i = threadIdx.x; i < half; i += blockDim.x) sincosf(pos * a.feed.inv_freq[i], &turn[i].x, &turn[i].y);
+        __syncthreads();
+    }
     const int nq = a.H * (a.dks / 4), nv = a.H * (a.dvs / 4);
     for (int idx = threadIdx.x; idx < 2 * nq + nv; idx += blockDim.x) {
         const int which = idx < nq ? 0 : idx < 2 * nq ? 1 : 2;
@@ -170,7 +215,17 @@ __global__ __launch_bounds__(256) void lightning_prepare_kernel(LcPrepArgs a) {
         const T* src = row + (which == 0 ? a.q_col : which == 1 ? a.k_col : a.v_col) + (size_t)h * width + r;
         float e[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) e[i] = r + i < width ? la_silu(to_f32(src[i])) : 0.f;
+        for (int i = 0; i < 4; ++i) {
+            e[i] = r + i < width ? la_act(to_f32(src[i]), a.feed.silu) : 0.f;
+            if (which == 2) continue;
+            if (r + i < 2 * half) {                          // dimension d turns with d + half, or with d - half behind it
+                const bool first = r + i < half;
+                const float2 sc = turn[first ? r + i : r + i - half];
+                const float other = la_act(to_f32(src[first ? i + half : i - half]), a.feed.silu);
+                e[i] = first ? e[i] * sc.y - other * sc.x : e[i] * sc.y + other * sc.x;
+            }
+            if (which == 1) e[i] *= a.feed.k_scale;
+        }
         float* dst = (which == 0 ? a.q : which == 1 ? a.k : a.v) + ((size_t)h * a.T + t) * ws + r;
         *reinterpret_cast<float4*>(dst) = make_float4(e[0], e[1], e[2], e[3]);
     }
@@ -192,7 +247,7 @@ __global__ __launch_bounds__(LA_THREADS) void lightning_chunk_kernel(LaArgs a) {
     constexpr int DKP = 64 * RT, CB = 16 * NCT;
     constexpr int LDQ = DKP + 4, LDV = CB + 4, LDA = LC_C + 4;     // rows 16 bytes apart from a multiple of 128: few bank conflicts
     extern __shared__ __align__(16) float la_smem[];
-    float* Q_s = la_smem;                                 // [LC_C][LDQ]   silu(q), rows from the chunk's tokens on zero
+    float* Q_s = la_smem;                                 // [LC_C][LDQ]   q, rows from the chunk's tokens on zero
     float* K_s = Q_s + LC_C * LDQ;                        // [LC_C][LDQ]
     float* V_s = K_s + LC_C * LDQ;                        // [LC_C][LDV]
     float* A_s = V_s + LC_C * LDV;                        // [LC_C][LDA]   decayed scores, the causal half
@@ -400,8 +455,9 @@ static int lc_launch(const LaArgs& a, int n_seqs, hipStream_t s) {
     return bn_launch_status();
 }
 
-static int lc_dispatch(int dtype, LaArgs& a, int n_seqs, int n_rows, float* prepared, hipStream_t s) {
+static int lc_dispatch(int dtype, LaArgs& a, int n_seqs, int n_rows, const int* positions, float* prepared, hipStream_t s) {
     LcPrepArgs p;
+    p.feed = a.feed; p.positions = positions;
     p.x = a.x; p.T = n_rows; p.ld = a.ld; p.q_col = a.q_col; p.k_col = a.k_col; p.v_col = a.v_col; p.H = a.H; p.dk = a.dk; p.dv = a.dv;
     p.dks = (a.dk + 3) / 4 * 4; p.dvs = (a.dv + 3) / 4 * 4;
     p.q = prepared; p.k = p.q + (size_t)a.H * n_rows * p.dks; p.v = p.k + (size_t)a.H * n_rows * p.dks;
@@ -430,9 +486,13 @@ extern "C" int bn_lightning_prefers_chunks(int n_seqs, int H, int dk, int dv) {
 // x [T, ld] holds q at q_col, k at k_col (H dk wide each) and v at v_col (H dv wide); n_seqs: tiles, or rows of a decode step;
 // prepared: room for the chunked form's copy of q, k and v, n_rows H (2 dks + dvs) floats with n_rows the rows of x and dks,
 // dvs the widths rounded up to a multiple of 4; null: the chain form also where the chunked form would run
+// silu: 1, q, k and v pass a silu, 0, they come as projected; inv_freq [rope_dims / 2] or null: the rotation of q and k, whose
+// positions the chunked form takes from positions [n_rows]; k_scale multiplies k
 extern "C" int bn_lightning_scan(int dtype, const void* x, int ld, int q_col, int k_col, int v_col, const float* decay, float* o,
                                  float* state, long long state_stride, const int* tiles, int n_seqs, const int* seq_lens,
-                                 const int* slot_ids, int H, int dk, int dv, int n_rows, float* prepared, hipStream_t s) {
+                                 const int* slot_ids, int H, int dk, int dv, int n_rows, float* prepared, int silu,
+                                 const float* inv_freq, int rope_dims, const int* positions, float k_scale, hipStream_t s) {
+    if (inv_freq ? (rope_dims < 2 || rope_dims % 2 || rope_dims > dk) : rope_dims != 0) return BN_ERR_ARG;
     if (n_seqs <= 0 || H <= 0 || !bn_lightning_supports(dk, dv) || !x || !decay || !o || !state || !slot_ids) return BN_ERR_ARG;
     if ((!tiles && !seq_lens) || state_stride < (long long)H * dk * dv || q_col < 0 || k_col < 0 || v_col < 0) return BN_ERR_ARG;
     if (ld < q_col + H * dk || ld < k_col + H * dk || ld < v_col + H * dv) return BN_ERR_ARG;
@@ -440,10 +500,11 @@ extern "C" int bn_lightning_scan(int dtype, const void* x, int ld, int q_col, in
     a.x = x; a.o = o; a.decay = decay; a.state = state; a.state_stride = (size_t)state_stride; a.tiles = tiles;
     a.seq_lens = seq_lens; a.slot_ids = slot_ids; a.ld = ld; a.q_col = q_col; a.k_col = k_col; a.v_col = v_col;
     a.H = H; a.dk = dk; a.dv = dv;
+    a.feed.silu = silu ? 1 : 0; a.feed.rope_dims = rope_dims; a.feed.inv_freq = inv_freq; a.feed.k_scale = k_scale;
     if (dtype != BN_DT_F32 && dtype != BN_DT_BF16) return BN_ERR_DTYPE;
     if (tiles && prepared && bn_lightning_chunked(dk, dv)) {
-        if (n_rows <= 0 || (uintptr_t)prepared % 16 != 0) return BN_ERR_ARG;
-        return lc_dispatch(dtype, a, n_seqs, n_rows, prepared, s);
+        if (n_rows <= 0 || (uintptr_t)prepared % 16 != 0 || (inv_freq && !positions)) return BN_ERR_ARG;
+        return lc_dispatch(dtype, a, n_seqs, n_rows, positions, prepared, s);
     }
     const int rpt = dk <= 32 ? 8 : dk <= 64 ? 16 : dk <= 128 ? 32 : 64;
     const size_t smem = (size_t)LA_TC * (2 * rpt * LA_RG + LA_CB + LA_RG * LA_CB) * sizeof(float);

@@ -5,7 +5,9 @@
 //   bn_moe_route     router logits z = W_r h (+ a bias per expert) in float32 (one workgroup a token), scores sigmoid(z) or softmax(z), the top_k
 //                    largest (ties: the lower index; with a choice bias the largest score + bias, the weights staying the
 //                    plain scores), optionally divided by their sum (+ floor), times a constant -> expert ids and weights
-//                    [T, top_k]; optionally also sigmoid(w_g . h) per token, the gate of a shared expert
+//                    [T, top_k]; optionally also sigmoid(w_g . h) per token, the gate of a shared expert.  With groups the
+//                    experts fall into groups of neighbours, a group ranks by its best member, and only members of the
+//                    best `keep` groups (ties: the lower index) can be chosen
 //   bn_gated_unit    rows of stacked (gate | up) products -> the clamped unit, optionally times a factor per row
 //   bn_moe_experts   for every (token, choice) pair: y = W_down[e] act(W_up[e] (w h)) when the weight multiplies the
 //                    expert's input, w * W_down[e] act(W_up[e] h) when it multiplies the output; a pair reads its expert's
@@ -14,6 +16,7 @@
 //                    see them.
 //   bn_moe_group     (bf16, steps of many rows) pairs ordered by expert, tiles of rows of one expert each, and the inputs
 //                    gathered in that order, for the grouped matrix products of gemm_mfma.hip
+// Experts from E on are identity experts: they have no matrices, and their output is the token's own row times the weight.
 // The outputs of a token's choices land in slab j of y [top_k, T, D] (float32) and are added by whoever consumes y.
 #include "common.h"
 #include <math.h>
@@ -34,6 +37,7 @@ struct RouteArgs {
     const float* gate_w;      // [D]: gate_out[t] = sigmoid(gate_w . h); null: none
     float* gate_out;          // [T]
     float floor, scale;       // weights = score / (sum of the chosen + floor) (when renorm) * scale
+    int groups, keep;         // groups > 1: E / groups neighbours a group, the best `keep` groups stay in the choice
 };
 
 #define MOE_ROUTE_THREADS 256
@@ -96,6 +100,35 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
             }
         }
     }
+    if (a.groups > 1) {
+        // the ranking values (the logits rank as their scores do) meet in shared memory, where this wave alone is left: a
+        // lane takes groups lane, lane + 64, ..., forms their best members' values, then counts the groups ahead of each
+        float* rank = zs;
+        float* best = zs + a.E;
+        const int size = a.E / a.groups;
+#pragma unroll
+        for (int j = 0; j < MOE_PER_LANE; ++j)
+            if (lane + BN_WAVE * j < a.E) rank[lane + BN_WAVE * j] = z[j];
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+        for (int g = lane; g < a.groups; g += BN_WAVE) {
+            float m = -INFINITY;
+            for (int i = 0; i < size; ++i) m = fmaxf(m, rank[g * size + i]);
+            best[g] = m;
+        }
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (int j = 0; j < MOE_PER_LANE; ++j) {
+            const int e = lane + BN_WAVE * j;
+            if (e >= a.E) continue;
+            const int g = e / size;
+            const float m = best[g];
+            int ahead = 0;
+            for (int o = 0; o < a.groups; ++o) ahead += (best[o] > m || (best[o] == m && o < g)) ? 1 : 0;
+            if (ahead >= a.keep) z[j] = -INFINITY;
+        }
+    }
     float total = 0.f, mine_w = 0.f;
     int mine_id = 0;
     for (int k = 0; k < a.K; ++k) {
@@ -135,16 +168,19 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
 
 extern "C" int bn_moe_route(int dtype, const void* h, int ld, const float* wr, int* ids, float* wts, int n_tokens, int D, int E,
                             int K, int scoring, int renorm, const float* bias, float floor, float scale, const float* gate_w,
-                            float* gate_out, const float* zbias, hipStream_t s) {
+                            float* gate_out, const float* zbias, int groups, int keep, hipStream_t s) {
+    // groups of equal size, of which the kept ones hold at least the chosen number
+    if (groups < 1 || E % groups || keep < 1 || keep > groups || (long long)keep * (E / groups) < K) return BN_ERR_ARG;
     if ((gate_w == nullptr) != (gate_out == nullptr) || ((uintptr_t)gate_w & 15) || !(floor >= 0.f)) return BN_ERR_ARG;
     if (n_tokens <= 0 || D <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || K <= 0 || K > E || ld < D || !h || !wr || !ids || !wts)
         return BN_ERR_ARG;
     if (scoring != MOE_SCORE_SIGMOID && scoring != MOE_SCORE_SOFTMAX) return BN_ERR_ARG;
-    if ((size_t)(D + 4 + E) * sizeof(float) > 64 * 1024 || ((uintptr_t)wr & 15)) return BN_ERR_ARG;
+    if ((size_t)(D + 4 + E + groups) * sizeof(float) > 64 * 1024 || ((uintptr_t)wr & 15)) return BN_ERR_ARG;
     RouteArgs a;
     a.h = h; a.wr = wr; a.ids = ids; a.wts = wts; a.ld = ld; a.D = D; a.E = E; a.K = K; a.scoring = scoring; a.renorm = renorm ? 1 : 0;
     a.bias = bias; a.zbias = zbias; a.gate_w = gate_w; a.gate_out = gate_out; a.floor = floor; a.scale = scale;
-    const size_t shm = (size_t)(((D + 3) & ~3) + E) * sizeof(float);
+    a.groups = groups; a.keep = keep;
+    const size_t shm = (size_t)(((D + 3) & ~3) + E + groups) * sizeof(float);
     if (dtype == BN_DT_F32) hipLaunchKernelGGL(moe_route_kernel<float>, dim3(n_tokens), dim3(MOE_ROUTE_THREADS), shm, s, a);
     else if (dtype == BN_DT_BF16) hipLaunchKernelGGL(moe_route_kernel<bf16>, dim3(n_tokens), dim3(MOE_ROUTE_THREADS), shm, s, a);
     else return BN_ERR_DTYPE;
@@ -167,7 +203,7 @@ struct PairArgs {
     const float* wts;         // [T, K]
     float* hidden;            // [T K, F] float32 holding values of the activations' type
     float* y;                 // [K, T, D]
-    int ld, T, D, F, K, act, weight_on_input;      // T: the rows of a slab of y
+    int ld, T, D, F, K, E, act, weight_on_input;   // T: the rows of a slab of y; ids from E on: identity experts
     int gated;                // w_up is [E, 2 F, D]: F gate rows, then F up rows; hidden = the clamped unit of the two
     float limit, slope, shift;
 };
@@ -212,6 +248,7 @@ __global__ __launch_bounds__(MOE_PAIR_THREADS) void moe_pair_up_kernel(PairArgs 
     const int pair = blockIdx.y, t = pair / a.K;
     const int lane = threadIdx.x & (BN_WAVE - 1), wave = threadIdx.x / BN_WAVE;
     const int e = a.ids[pair];
+    if (e >= a.E) return;                                // an identity expert: nothing to multiply
     const float in_scale = a.weight_on_input ? a.wts[pair] : 1.0f;
     const T* h = reinterpret_cast<const T*>(a.h) + (size_t)t * a.ld;
     for (int d = threadIdx.x; d < a.D; d += MOE_PAIR_THREADS) xs[d] = to_f32(from_f32<T>(to_f32(h[d]) * in_scale));
@@ -260,6 +297,13 @@ __global__ __launch_bounds__(MOE_PAIR_THREADS) void moe_pair_down_kernel(PairArg
     const int lane = threadIdx.x & (BN_WAVE - 1), wave = threadIdx.x / BN_WAVE;
     const int e = a.ids[pair];
     const float out_scale = a.weight_on_input ? 1.0f : a.wts[pair];
+    if (e >= a.E) {                                      // an identity expert: the token's row times the weight
+        const T* h = reinterpret_cast<const T*>(a.h) + (size_t)t * a.ld;
+        float* yi = a.y + ((size_t)j * a.T + t) * a.D;
+        const int d = blockIdx.x * MOE_PAIR_ROWS + threadIdx.x;
+        if (threadIdx.x < MOE_PAIR_ROWS && d < a.D) yi[d] = to_f32(h[d]) * a.wts[pair];
+        return;
+    }
     for (int f = threadIdx.x; f < a.F; f += MOE_PAIR_THREADS) hid[f] = a.hidden[(size_t)pair * a.F + f];
     __syncthreads();
     const T* wd = reinterpret_cast<const T*>(a.w_down) + (size_t)e * a.D * a.F;
@@ -281,15 +325,15 @@ __global__ __launch_bounds__(MOE_PAIR_THREADS) void moe_pair_down_kernel(PairArg
 // hidden: float32 work space [n_tokens K, F]; y_rows: the rows of a slab of y (>= n_tokens: the call may take a run of a
 // step's tokens, y then points at the run's first row of slab 0)
 extern "C" int bn_moe_experts(int dtype, const void* h, int ld, const void* w_up, const void* w_down, const int* ids,
-                              const float* wts, float* y, float* hidden, int n_tokens, int y_rows, int D, int F, int K, int act,
+                              const float* wts, float* y, float* hidden, int n_tokens, int y_rows, int D, int F, int E, int K, int act,
                               int weight_on_input, int gated, float limit, float slope, float shift, hipStream_t s) {
-    if (n_tokens <= 0 || y_rows < n_tokens || D <= 0 || F <= 0 || K <= 0 || ld < D) return BN_ERR_ARG;
+    if (n_tokens <= 0 || y_rows < n_tokens || D <= 0 || F <= 0 || E <= 0 || K <= 0 || ld < D) return BN_ERR_ARG;
     if (gated ? !(limit > 0.f) : (act < 0 || act >= BN_UNARY_KINDS)) return BN_ERR_ARG;
     if (!h || !w_up || !w_down || !ids || !wts || !y || !hidden) return BN_ERR_ARG;
     if ((size_t)D * sizeof(float) > 64 * 1024 || (size_t)F * sizeof(float) > 64 * 1024 || (size_t)n_tokens * K > 65535) return BN_ERR_ARG;
     PairArgs a;
     a.h = h; a.w_up = w_up; a.w_down = w_down; a.ids = ids; a.wts = wts; a.y = y; a.hidden = hidden;
-    a.ld = ld; a.T = y_rows; a.D = D; a.F = F; a.K = K; a.act = act; a.weight_on_input = weight_on_input ? 1 : 0;
+    a.ld = ld; a.T = y_rows; a.D = D; a.F = F; a.K = K; a.E = E; a.act = act; a.weight_on_input = weight_on_input ? 1 : 0;
     a.gated = gated ? 1 : 0; a.limit = limit; a.slope = slope; a.shift = shift;
     const dim3 block(MOE_PAIR_THREADS);
     const dim3 up((F + MOE_PAIR_ROWS - 1) / MOE_PAIR_ROWS, n_tokens * K), down((D + MOE_PAIR_ROWS - 1) / MOE_PAIR_ROWS, n_tokens * K);
@@ -310,14 +354,14 @@ extern "C" int bn_moe_experts(int dtype, const void* h, int ld, const void* w_up
 // memory, so the launches do not depend on the routing.
 #define MOE_PLAN_THREADS 1024
 
-// order [T K]: the pairs (t K + j) by expert; tiles [max_tiles][3] = expert, first place in `order`, rows; n_tiles [1]
+// order [T K]: the pairs (t K + j) by expert, those of identity experts (ids from E on) behind all others and in no tile; tiles [max_tiles][3] = expert, first place in `order`, rows; n_tiles [1]
 __global__ __launch_bounds__(MOE_PLAN_THREADS) void moe_plan_kernel(const int* __restrict__ ids, int n_pairs, int E, int tile_rows,
                                                                     int* __restrict__ order, int* __restrict__ tiles,
                                                                     int* __restrict__ n_tiles) {
-    __shared__ int count[MOE_MAX_EXPERTS], first[MOE_MAX_EXPERTS + 1], tile0[MOE_MAX_EXPERTS + 1];
-    for (int e = threadIdx.x; e < E; e += blockDim.x) count[e] = 0;
+    __shared__ int count[MOE_MAX_EXPERTS + 1], first[MOE_MAX_EXPERTS + 1], tile0[MOE_MAX_EXPERTS + 1];
+    for (int e = threadIdx.x; e <= E; e += blockDim.x) count[e] = 0;
     __syncthreads();
-    for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) atomicAdd(&count[ids[p]], 1);
+    for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) atomicAdd(&count[min(ids[p], E)], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int at = 0, tl = 0;
@@ -337,25 +381,39 @@ __global__ __launch_bounds__(MOE_PLAN_THREADS) void moe_plan_kernel(const int* _
         }
         count[e] = 0;                                    // now the cursor of the scatter
     }
+    if (threadIdx.x == 0) count[E] = 0;
     __syncthreads();
     // the places inside an expert's run are handed out in whatever order the lanes arrive: a row's result does not depend
     // on its place
     for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) {
-        const int e = ids[p];
+        const int e = min(ids[p], E);
         order[first[e] + atomicAdd(&count[e], 1)] = p;
     }
 }
 
 // xg[place] = h[token of the pair at that place] (times the pair's weight, rounded to bf16, when scale_input); row_map[place]
 // = the pair's row of y seen as [K T, D]; row_scale[place] = the pair's weight.  One workgroup a place, 16 bytes a thread.
+// The pair of an identity expert (ids from E on) has its result here: its row of y is the token's row times the weight.
 __global__ __launch_bounds__(256) void moe_gather_kernel(const bf16* __restrict__ h, int ld, const int* __restrict__ order,
                                                          const float* __restrict__ wts, bf16* __restrict__ xg,
                                                          int* __restrict__ row_map, float* __restrict__ row_scale, int T, int D,
-                                                         int K, int scale_input) {
+                                                         int K, int scale_input, const int* __restrict__ ids, int E,
+                                                         float* __restrict__ y) {
     const int place = blockIdx.x, pair = order[place], t = pair / K, j = pair - t * K;
     const float w = wts[pair];
     if (threadIdx.x == 0) { row_map[place] = j * T + t; row_scale[place] = w; }
     const bf16* src = h + (size_t)t * ld;
+    if (ids[pair] >= E) {
+        float* yr = y + ((size_t)j * T + t) * D;
+        for (int d = 8 * threadIdx.x; d < D; d += 8 * 256) {
+            const uint4 p = *reinterpret_cast<const uint4*>(src + d);
+            *reinterpret_cast<float4*>(yr + d) = make_float4(bf16lo_to_f32(p.x) * w, bf16hi_to_f32(p.x) * w,
+                                                             bf16lo_to_f32(p.y) * w, bf16hi_to_f32(p.y) * w);
+            *reinterpret_cast<float4*>(yr + d + 4) = make_float4(bf16lo_to_f32(p.z) * w, bf16hi_to_f32(p.z) * w,
+                                                                 bf16lo_to_f32(p.w) * w, bf16hi_to_f32(p.w) * w);
+        }
+        return;
+    }
     bf16* dst = xg + (size_t)place * D;
     for (int d = 8 * threadIdx.x; d < D; d += 8 * 256) {
         uint4 p = *reinterpret_cast<const uint4*>(src + d);
@@ -375,11 +433,12 @@ extern "C" int bn_moe_grouped_tiles(int n_pairs, int E, int tile_rows) {
     return tile_rows > 0 ? (n_pairs + tile_rows - 1) / tile_rows + E : 0;
 }
 
+// y: float32 [K, n_tokens, D], of which the identity experts' rows are written here
 // work: int32 [2 n_pairs + 3 max_tiles + 1] = order, row_map, tiles, n_tiles; row_scale: float32 [n_pairs]; xg: bf16 [n_pairs, D]
 extern "C" int bn_moe_group(const void* h, int ld, const int* ids, const float* wts, int* work, float* row_scale, void* xg,
-                            int n_tokens, int D, int E, int K, int tile_rows, int scale_input, hipStream_t s) {
+                            int n_tokens, int D, int E, int K, int tile_rows, int scale_input, float* y, hipStream_t s) {
     if (n_tokens <= 0 || K <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || D <= 0 || D % 8 || ld < D || ld % 8 || tile_rows <= 0) return BN_ERR_ARG;
-    if (!h || !ids || !wts || !work || !row_scale || !xg || (((uintptr_t)h | (uintptr_t)xg) & 15)) return BN_ERR_ARG;
+    if (!h || !ids || !wts || !work || !row_scale || !xg || !y || (((uintptr_t)h | (uintptr_t)xg | (uintptr_t)y) & 15)) return BN_ERR_ARG;
     const int n_pairs = n_tokens * K, max_tiles = bn_moe_grouped_tiles(n_pairs, E, tile_rows);
     int* order = work;
     int* row_map = work + n_pairs;
@@ -387,7 +446,7 @@ extern "C" int bn_moe_group(const void* h, int ld, const int* ids, const float* 
     int* n_tiles = tiles + 3 * max_tiles;
     hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(MOE_PLAN_THREADS), 0, s, ids, n_pairs, E, tile_rows, order, tiles, n_tiles);
     hipLaunchKernelGGL(moe_gather_kernel, dim3(n_pairs), dim3(256), 0, s, (const bf16*)h, ld, order, wts, (bf16*)xg, row_map,
-                       row_scale, n_tokens, D, K, scale_input ? 1 : 0);
+                       row_scale, n_tokens, D, K, scale_input ? 1 : 0, ids, E, y);
     return bn_launch_status();
 }
 

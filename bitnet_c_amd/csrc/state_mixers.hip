@@ -374,7 +374,7 @@ extern "C" int bn_wkv_scan(int dtype, const void* r, int ldr, const void* k, int
 }
 
 // ---- per-head RMS of the recurrence's output, its weight and the gate -----------------------------------------------
-// one wave per (row, head): y = o / sqrt(mean(o^2) + eps) * weight * silu(gate)
+// one wave per (row, head): y = o / sqrt(mean(o^2) + eps) * weight * silu(gate); weight null: 1
 template <typename T>
 __global__ __launch_bounds__(BN_WAVE) void head_norm_gate_kernel(T* __restrict__ y, const float* __restrict__ o,
                                                                   const T* __restrict__ gate, int ldg,
@@ -387,13 +387,14 @@ __global__ __launch_bounds__(BN_WAVE) void head_norm_gate_kernel(T* __restrict__
     const float f = 1.0f / sqrtf(ss / (float)dv + eps);
     for (int e = lane; e < dv; e += BN_WAVE) {
         const float g = to_f32(gate[(size_t)t * ldg + (size_t)head * dv + e]);
-        y[((size_t)t * H + head) * dv + e] = from_f32<T>(ov[e] * f * weight[(size_t)head * dv + e] * bn_unary_act(g, BN_UNARY_SILU));
+        const float w = weight ? weight[(size_t)head * dv + e] : 1.0f;
+        y[((size_t)t * H + head) * dv + e] = from_f32<T>(ov[e] * f * w * bn_unary_act(g, BN_UNARY_SILU));
     }
 }
 
 extern "C" int bn_head_norm_gate(int dtype, void* y, const float* o, const void* gate, int ldg, const float* weight,
                                  int n_tokens, int H, int dv, float eps, hipStream_t s) {
-    if (n_tokens <= 0 || H <= 0 || dv <= 0 || !y || !o || !gate || !weight || ldg < H * dv) return BN_ERR_ARG;
+    if (n_tokens <= 0 || H <= 0 || dv <= 0 || !y || !o || !gate || ldg < H * dv) return BN_ERR_ARG;
     const dim3 grid(n_tokens, H);
     if (dtype == BN_DT_F32)
         hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(BN_WAVE), 0, s, (float*)y, o, (const float*)gate, ldg, weight, H, dv, eps);

@@ -65,21 +65,22 @@ _SIGNATURES = {
     },
     "latent": {
         "bn_latent_store": [c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
-                            c_int, c_int, c_float, c_int, c_void_p, c_float, c_void_p],
+                            c_int, c_int, c_float, c_int, c_void_p, c_float, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
+                            c_void_p],
         "bn_head_linear": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                           c_void_p],
+                           c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_void_p],
         "bn_sigmoid_gate": [c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
-        "bn_rope_heads": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p],
+        "bn_rope_heads": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
     },
     "moe": {
         "bn_moe_route": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                         c_void_p, c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p],
+                         c_void_p, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
         "bn_moe_experts": [c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
-                           c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_void_p],
+                           c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_void_p],
         "bn_gated_unit": [c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_float, c_float, c_void_p],
         "bn_moe_grouped_tiles": [c_int, c_int, c_int],
         "bn_moe_group": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                         c_int, c_void_p],
+                         c_int, c_void_p, c_void_p],
     },
     "attn_mfma_general": {
         "bn_attn_general_supports": [c_int, c_int],
@@ -110,12 +111,17 @@ _SIGNATURES = {
         "bn_gla_scan_pieces": [c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p,
                                c_int, c_void_p, c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_void_p, c_void_p, c_void_p],
     },
+    "twin_norm": {
+        "bn_twin_norm": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_float, c_void_p, c_int,
+                         c_int, c_void_p],
+    },
     "lightning": {
         "bn_lightning_supports": [c_int, c_int],
         "bn_lightning_chunked": [c_int, c_int],
         "bn_lightning_prefers_chunks": [c_int, c_int, c_int, c_int],
         "bn_lightning_scan": [c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p,
-                              c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p],
+                              c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p,
+                              c_float, c_void_p],
         "bn_row_norm_gate": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_int, c_void_p],
     },
     "state_mixers": {
@@ -1142,6 +1148,8 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
 
 
 MAX_HEAD_DIM = _build.header_constant("BN_MAX_HEAD_DIM")    # the attention kernels take every even head size up to this
+MAX_LATENT_KEY = _build.header_constant("BN_MAX_LATENT_KEY")       # and the vector kernel keys and values up to these widths,
+MAX_LATENT_VALUE = _build.header_constant("BN_MAX_LATENT_VALUE")   # where a latent is the one head of the cache
 
 
 def _pow2_at_least(n: int) -> int:
@@ -1331,8 +1339,8 @@ def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pag
     T = qkv.shape[0]
     if H % Hkv or qkv.shape[1] < H * hs or out.shape != (T, H * vd) or not out.is_contiguous():
         raise KernelError(f"attention: qkv {tuple(qkv.shape)} / out {tuple(out.shape)} do not fit H={H} hs={hs} v_dim={vd}")
-    if vd % 2 or vd < 2 or vd > MAX_HEAD_DIM:
-        raise KernelError(f"attention: value width {vd} is not supported (even, at most {MAX_HEAD_DIM})")
+    if vd % 2 or vd < 2 or vd > MAX_LATENT_VALUE:
+        raise KernelError(f"attention: value width {vd} is not supported (even, at most {MAX_LATENT_VALUE})")
     sink_flag, sink_ptr = _sink_args(sink, H, "attention")
     extras = vd != hs or distance_bias is not None or bool(sink_flag) or keep_first != 0
     if keep_first < 0:
@@ -1341,8 +1349,8 @@ def attention(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pag
         raise KernelError("attention: another value width, a distance bias, kept first positions and a sink are the vector kernel's, which reads "
                           "pages with a row per position or transposed values")
     da, db = _distance_args(distance_bias, H, "attention")
-    if hs % 2 or hs < 2 or hs > MAX_HEAD_DIM:
-        raise KernelError(f"attention: head size {hs} is not supported (even, at most {MAX_HEAD_DIM})")
+    if hs % 2 or hs < 2 or hs > MAX_LATENT_KEY:
+        raise KernelError(f"attention: head size {hs} is not supported (even, at most {MAX_LATENT_KEY})")
     if not block_table.is_contiguous():
         raise KernelError("attention: block_table must be contiguous")
     decode = tiles is None
@@ -1512,20 +1520,36 @@ def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, H: int, Hkv: int, 
 GENERAL_PROMPT_TILE = 16       # query tokens of a tile of attention_general_prompt
 # BITNET_NO_GENERAL_MFMA=1 keeps the attention mixer's general form on the vector kernel in prompt steps too
 GENERAL_PROMPT_ON_MATRIX_CORES = os.environ.get("BITNET_NO_GENERAL_MFMA", "") in ("", "0")
-_GENERAL_SIZES = (32, 64, 96, 128, 256)        # key widths; values may also be 192 wide (a latent beside a rotated key part)
+_GENERAL_SIZES = (32, 64, 96, 128, 192, 256)   # key and value widths
+_GENERAL_LATENT_KEYS = (160, 192)              # key widths of a latent beside a rotated part: values 64 wide or more, no wider than the keys
 
 
 def attention_general_supported(dtype, hs: int, v_dim: int) -> bool:
     """Whether attention_general_prompt takes this type and these head sizes (bn_attn_general_supports, answered here so
     that asking loads no kernel)."""
-    return dtype == torch.bfloat16 and int(hs) in _GENERAL_SIZES and int(v_dim) in _GENERAL_SIZES + (192,)
+    if dtype != torch.bfloat16 or int(v_dim) not in _GENERAL_SIZES:
+        return False
+    return 64 <= int(v_dim) <= int(hs) if int(hs) in _GENERAL_LATENT_KEYS else int(hs) in _GENERAL_SIZES
+
+
+def latent_row_widths(rank: int, rot_dims: int):
+    """(width of a stored key row, of a stored value row) for a latent of `rank` numbers beside rot_dims rotated ones: the
+    next sizes that the matrix-core attention kernels take, the columns behind the numbers zero, where that makes neither
+    row more than a quarter wider; else the sizes themselves (the vector kernel's)."""
+    kw, vw = rank + rot_dims, rank
+    for v in _GENERAL_SIZES:
+        if vw <= v <= vw + vw // 4:
+            for k in sorted(set(_GENERAL_SIZES + _GENERAL_LATENT_KEYS)):
+                if kw <= k <= kw + kw // 4 and attention_general_supported(torch.bfloat16, k, v):
+                    return k, v
+    return kw, vw
 
 
 def attention_general_prompt(qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                              block_table: torch.Tensor, H: int, Hkv: int, hs: int, v_dim: int, scale: float, tiles: torch.Tensor,
                              *, distance_bias=None, sink: bool = False, window: int = 0, keep_first: int = 0, gate=None) -> None:
-    """Causal prompt attention on the matrix cores for what attention() leaves to the vector kernel: bf16, keys 32, 64,
-    96, 128 or 256 wide, values of a width of their own from the same list, a distance bias and a sink (as attention()'s),
+    """Causal prompt attention on the matrix cores for what attention() leaves to the vector kernel: bf16, keys and values of
+    the widths that attention_general_supported() takes, a distance bias and a sink (as attention()'s),
     a window (> 0: a query sees the last `window` positions, its own included, and the first keep_first positions).  gate: a
     bf16 tensor [T, H v_dim] (it may be columns of a wider one): the result times sigmoid(gate).  qkv's row stride is a multiple of 8.
     Pages: keys a row per position, values transposed.  tiles [n, 4] int32: (sequence, first row, rows <= 16, position of
@@ -1895,21 +1919,23 @@ def wkv_scan(r, k, v, d, w0, u, h, state, slot_ids, H: int, dk: int, dv: int, *,
     return o
 
 
-def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, H: int, dv: int, eps: float) -> torch.Tensor:
+def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], H: int, dv: int, eps: float) -> torch.Tensor:
     """o [T, H dv] float32, each head divided by its root mean square (eps inside the root), times weight [H dv]
-    (float32), times silu(gate) (gate [T, H dv] in the activations' type, which is the result's)."""
+    (float32; None: 1), times silu(gate) (gate [T, H dv] in the activations' type, which is the result's)."""
     require_gpu()
     _dev(o, "o", torch.float32, 2)
     _dev(gate, "gate", dims=2)
-    _dev(weight, "weight", torch.float32, 1)
     T = o.shape[0]
-    if o.shape[1] != H * dv or not o.is_contiguous() or gate.shape != o.shape or weight.numel() != H * dv or not weight.is_contiguous():
+    if weight is not None:
+        _dev(weight, "weight", torch.float32, 1)
+    if o.shape[1] != H * dv or not o.is_contiguous() or gate.shape != o.shape or (
+            weight is not None and (weight.numel() != H * dv or not weight.is_contiguous())):
         raise KernelError("head_norm_gate: o and gate [T, H dv], weight [H dv]")
     y = torch.empty((T, H * dv), dtype=gate.dtype, device=o.device)
     if T:
         _check(_fn("state_mixers", "bn_head_norm_gate")(_code(gate.dtype), y.data_ptr(), o.data_ptr(), gate.data_ptr(),
-                                                        _rows(gate, "gate"), weight.data_ptr(), T, H, dv, float(eps), _stream()),
-               "head_norm_gate")
+                                                        _rows(gate, "gate"), weight.data_ptr() if weight is not None else None, T, H, dv,
+                                                        float(eps), _stream()), "head_norm_gate")
     return y
 
 
@@ -1958,7 +1984,9 @@ def lightning_chunked(dk: int, dv: int) -> bool:
 
 
 def lightning_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, decay: torch.Tensor, state: torch.Tensor, slot_ids,
-                   H: int, dk: int, dv: int, *, tiles=None, seq_lens=None, chain: Optional[bool] = None) -> torch.Tensor:
+                   H: int, dk: int, dv: int, *, tiles=None, seq_lens=None, chain: Optional[bool] = None, silu: bool = True,
+                   inv_freq: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
+                   k_scale: float = 1.0) -> torch.Tensor:
     """Linear attention with a fixed decay per head over every sequence of a step; float32 [T, H dv].  x [T, >= ...] in
     the activations' type holds the projections side by side: queries at column q_col and keys at k_col (H dk wide),
     values at v_col (H dv wide); each passes silu in float32.  decay [H] float32.  state [slots, >= H dk dv] float32, the
@@ -1966,7 +1994,10 @@ def lightning_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, decay: t
         S <- decay S + k_t v_t^T;  o_t = S^T q_t.
     A prompt step (tiles) of a key width that lightning_chunked() takes can run the same sums chunk by chunk on the matrix
     cores, in float32, instead of token by token as decode steps do.  chain: True the token-by-token kernel, False the
-    chunks where they can be, None whichever is the faster for this many sequences and heads."""
+    chunks where they can be, None whichever is the faster for this many sequences and heads.
+    silu False: q, k and v enter as projected.  inv_freq [n <= dk / 2] float32 (with positions [T] int32, the rows' positions
+    once more): dimension i < n of every query and key head turns with dimension i + n by position * inv_freq[i].
+    k_scale multiplies the keys."""
     require_gpu()
     _dev(x, "x", dims=2)
     _dev(decay, "decay", torch.float32, 1)
@@ -1983,17 +2014,26 @@ def lightning_scan(x: torch.Tensor, q_col: int, k_col: int, v_col: int, decay: t
     tl, n_seqs, sl = _seq_args(tiles, seq_lens, "lightning_scan")
     if tiles is None and n_seqs != T:
         raise KernelError("lightning_scan: a decode step has one length per row")
+    rope_dims = 0
+    if inv_freq is not None:
+        _dev(inv_freq, "inv_freq", torch.float32, 1)
+        _dev(positions, "positions", torch.int32, 1)
+        rope_dims = 2 * inv_freq.numel()
+        if not 2 <= rope_dims <= dk or not inv_freq.is_contiguous() or positions.numel() != T or not positions.is_contiguous():
+            raise KernelError(f"lightning_scan: {rope_dims} rotated dimensions of {dk}, positions {tuple(positions.shape)} for {T} rows")
     o = torch.empty((T, H * dv), dtype=torch.float32, device=x.device)
     if T and n_seqs:
         prepared = None
         if tiles is not None and chain is not True and lightning_chunked(dk, dv) and (
                 chain is False or _fn("lightning", "bn_lightning_prefers_chunks")(n_seqs, H, dk, dv)):
-            # the chunked form's own copy of the step's q, k and v: silu applied, float32, head by head
+            # the chunked form's own copy of the step's q, k and v: what they pass applied, float32, head by head
             prepared = torch.empty(H * T * (2 * ((dk + 3) // 4 * 4) + (dv + 3) // 4 * 4), dtype=torch.float32, device=x.device)
         _check(_fn("lightning", "bn_lightning_scan")(_code(x.dtype), x.data_ptr(), ld, int(q_col), int(k_col), int(v_col),
                                                      decay.data_ptr(), o.data_ptr(), state.data_ptr(), stride, tl, n_seqs, sl,
                                                      slot_ids.data_ptr(), H, dk, dv, T,
-                                                     prepared.data_ptr() if prepared is not None else None, _stream()),
+                                                     prepared.data_ptr() if prepared is not None else None, int(bool(silu)),
+                                                     inv_freq.data_ptr() if rope_dims else None, rope_dims,
+                                                     positions.data_ptr() if rope_dims else None, float(k_scale), _stream()),
                "lightning_scan")
     return o
 
@@ -2062,13 +2102,16 @@ def add_normed_rmsnorm(x: torch.Tensor, delta, out_weight: torch.Tensor, out_eps
 
 def latent_store(x: torch.Tensor, col: int, rank: int, weight: torch.Tensor, eps: float, positions, seq_index, block_table,
                  k_pages: torch.Tensor, v_pages: torch.Tensor, *, rot_dims: int = 0, inv_freq: Optional[torch.Tensor] = None,
-                 rot_mult: float = 1.0) -> None:
+                 rot_mult: float = 1.0, interleaved: bool = False, row_widths=None, query=None):
     """Columns col .. col + rank of every row of x under an RMSNorm (weight [rank] float32, eps inside the root, float32
     arithmetic), stored at the row's position of its sequence's pages: as a key row ([pages, 1, PAGE, rank]) and into the
     transposed value page ([pages, 1, rank, PAGE]).  Rows with position < 0 store nothing.
     rot_dims > 0: the next rot_dims columns of x are one more key part, not normed, dimension i turned with dimension
-    i + rot_dims / 2 by position * inv_freq[i] (cosine and sine times rot_mult); a key row is then rank + rot_dims wide
-    and holds it behind the latent, the value page stays rank wide."""
+    i + rot_dims / 2 (interleaved: 2i with 2i + 1) by position * inv_freq[i] (cosine and sine times rot_mult); a key row is
+    then rank + rot_dims wide and holds it behind the latent, the value page stays rank wide.  row_widths (kw, vw): the
+    stored rows are that wide instead, the columns behind the numbers zero.
+    query = (column, weight [n] float32): columns column .. column + n of every row under the same kind of norm, returned
+    as [T, n] in x's type (every row, also those that store nothing)."""
     require_gpu()
     _dev(x, "x", dims=2)
     _dev(weight, "weight", torch.float32, 1)
@@ -2077,7 +2120,17 @@ def latent_store(x: torch.Tensor, col: int, rank: int, weight: torch.Tensor, eps
     _dev(block_table, "block_table", torch.int32, 2)
     T = x.shape[0]
     rot_dims = int(rot_dims)
-    _check_pages(k_pages, v_pages, 1, rank + rot_dims, x.dtype, True, False, rank)
+    kw, vw = (int(w) for w in row_widths) if row_widths is not None else (rank + rot_dims, rank)
+    if kw < rank + rot_dims or vw < rank:
+        raise KernelError(f"latent_store: stored rows of {kw} and {vw} do not hold {rank} + {rot_dims} numbers")
+    _check_pages(k_pages, v_pages, 1, kw, x.dtype, True, False, vw)
+    q_col, q_weight, q_out = 0, None, None
+    if query is not None:
+        q_col, q_weight = int(query[0]), query[1]
+        _dev(q_weight, "query weight", torch.float32, 1)
+        if q_col < 0 or x.shape[1] < q_col + q_weight.numel() or not q_weight.is_contiguous():
+            raise KernelError(f"latent_store: x {tuple(x.shape)} does not hold {q_weight.numel()} query columns from {q_col}")
+        q_out = torch.empty((T, q_weight.numel()), dtype=x.dtype, device=x.device)
     if rot_dims:
         _dev(inv_freq, "inv_freq", torch.float32, 1)
         if rot_dims % 2 or inv_freq.numel() != rot_dims // 2 or not inv_freq.is_contiguous():
@@ -2086,19 +2139,22 @@ def latent_store(x: torch.Tensor, col: int, rank: int, weight: torch.Tensor, eps
             or seq_index.numel() != T or not block_table.is_contiguous()):
         raise KernelError(f"latent_store: x {tuple(x.shape)} / columns {col}..{col + rank} / weight {tuple(weight.shape)} do not fit")
     if T == 0:
-        return
+        return q_out
     _check(_fn("latent", "bn_latent_store")(_code(x.dtype), x.data_ptr(), _rows(x, "x"), int(col), positions.data_ptr(),
                                             seq_index.data_ptr(), block_table.data_ptr(), block_table.shape[1],
                                             k_pages.data_ptr(), v_pages.data_ptr(), weight.data_ptr(), T, int(rank), float(eps),
                                             rot_dims, inv_freq.data_ptr() if rot_dims else None, float(rot_mult),
-                                            _stream()), "latent_store")
+                                            int(bool(interleaved)), kw, vw, q_col, q_weight.numel() if query is not None else 0,
+                                            q_weight.data_ptr() if query is not None else None,
+                                            q_out.data_ptr() if query is not None else None, _stream()), "latent_store")
+    return q_out
 
 
 def rope_heads(x: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor, H: int, head_stride: int, offset: int,
-               rot_dims: int, mult: float = 1.0) -> None:
+               rot_dims: int, mult: float = 1.0, interleaved: bool = False) -> None:
     """In place on x [T, >= (H - 1) head_stride + offset + rot_dims]: in every head (head h starts at column
-    h * head_stride) the rot_dims columns from `offset` on are rotated, dimension i with dimension i + rot_dims / 2, by
-    position * inv_freq[i]; cosine and sine times `mult`.  Rows with position < 0 are left alone."""
+    h * head_stride) the rot_dims columns from `offset` on are rotated, dimension i with dimension i + rot_dims / 2
+    (interleaved: 2i with 2i + 1), by position * inv_freq[i]; cosine and sine times `mult`.  Rows with position < 0 are left alone."""
     require_gpu()
     _dev(x, "x", dims=2)
     _dev(positions, "positions", torch.int32, 1)
@@ -2111,17 +2167,18 @@ def rope_heads(x: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor,
     if T:
         _check(_fn("latent", "bn_rope_heads")(_code(x.dtype), x.data_ptr(), _rows(x, "x"), positions.data_ptr(),
                                               inv_freq.data_ptr(), T, int(H), int(head_stride), int(offset), int(rot_dims),
-                                              float(mult), _stream()), "rope_heads")
+                                              float(mult), int(bool(interleaved)), _stream()), "rope_heads")
 
 
 HEAD_LINEAR_MAX_IN = 1792          # the kernel stages 8 rows of a head's input as float32 beside its partial sums in 64 KB of shared memory
 
 
 def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] = None, *,
-                allow_library: Optional[bool] = None, gate_per_head: bool = False) -> torch.Tensor:
+                allow_library: Optional[bool] = None, gate_per_head: bool = False, rotate=None) -> torch.Tensor:
     """A product per head: y[t, h, :] = x[t, h, :] . w[h] with x [T, H I] (rows contiguous), w [H, I, O] -> y [T, H O];
     with `gate` [T, H O] (rows contiguous) y is multiplied by sigmoid(gate) element by element, or, with gate_per_head,
     head h of y by sigmoid of the one number gate[t, h] (gate [T, H]).  float32 accumulation.
+    rotate = (positions, inv_freq, offset, mult, interleaved), without a gate: y as rope_heads() would leave it.
     bf16 with more than SKINNY_ROWS rows goes to the library's batched product (allow_library as linear's), everything else
     to a kernel that reads every head's matrix once for 8 rows."""
     require_gpu()
@@ -2136,6 +2193,16 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] =
         if tuple(gate.shape) != (T, H if gate_per_head else H * O):
             raise KernelError(f"head_linear: gate {tuple(gate.shape)} is not [{T}, {H if gate_per_head else H * O}]")
     group = O if gate_per_head else 1
+    rot = (None, None, 0, 0, 1.0, 0)
+    if rotate is not None:
+        positions, inv_freq, offset, mult, interleaved = rotate
+        _dev(positions, "positions", torch.int32, 1)
+        _dev(inv_freq, "inv_freq", torch.float32, 1)
+        if (gate is not None or positions.numel() != T or not positions.is_contiguous() or not inv_freq.is_contiguous()
+                or not 0 <= offset <= O - 2 * inv_freq.numel() or inv_freq.numel() < 1):
+            raise KernelError(f"head_linear: {2 * inv_freq.numel()} rotated columns from {offset} of {O}, positions "
+                              f"{tuple(positions.shape)} for {T} rows, gate {gate is not None}")
+        rot = (positions.data_ptr(), inv_freq.data_ptr(), int(offset), 2 * inv_freq.numel(), float(mult), int(bool(interleaved)))
     y = torch.empty((T, H * O), dtype=x.dtype, device=x.device)
     if T == 0:
         return y
@@ -2145,6 +2212,9 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] =
     if x.dtype == torch.bfloat16 and T > SKINNY_ROWS and allow_library:
         xv = x.as_strided((H, T, I), (I, ldx, 1))
         torch.bmm(xv, w, out=y.view(T, H, O).transpose(0, 1))
+        if rotate is not None:
+            positions, inv_freq, offset, mult, interleaved = rotate
+            rope_heads(y, positions, inv_freq, H, O, offset, 2 * inv_freq.numel(), mult, interleaved)
         if gate is not None:
             _check(_fn("latent", "bn_sigmoid_gate")(_code(y.dtype), y.data_ptr(), H * O, gate.data_ptr(), _rows(gate, "gate"),
                                                     group, T, H * O, _stream()), "sigmoid_gate")
@@ -2153,9 +2223,45 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] =
         raise KernelError(f"head_linear: a head's input of {I} values is above {HEAD_LINEAR_MAX_IN}")
     _check(_fn("latent", "bn_head_linear")(_code(x.dtype), x.data_ptr(), ldx, w.data_ptr(), y.data_ptr(), H * O,
                                            gate.data_ptr() if gate is not None else None,
-                                           _rows(gate, "gate") if gate is not None else 0, group, T, H, I, O, _stream()),
+                                           _rows(gate, "gate") if gate is not None else 0, group, T, H, I, O, *rot, _stream()),
            "head_linear")
     return y
+
+
+# --------------------------------------------------------------------------------------
+# a block whose two halves read the same stream (csrc/twin_norm.hip)
+# --------------------------------------------------------------------------------------
+
+def add_twin_rmsnorm(x: torch.Tensor, deltas, norms, out_dtype) -> list:
+    """x (float32, [T, D]) += the deltas in one pass: at most one tensor [T, D] of out_dtype and at most one PartialSums, in
+    this order.  norms: up to two (weight [D] float32, eps); the result is a list with the new rows of x under each, in
+    out_dtype."""
+    require_gpu()
+    _dev(x, "x", torch.float32, 2)
+    T, D = x.shape
+    y = [d for d in deltas if isinstance(d, torch.Tensor)]
+    parts = [d for d in deltas if isinstance(d, PartialSums)]
+    if len(y) > 1 or len(parts) > 1 or len(y) + len(parts) != len(deltas) or len(norms) > 2 or not x.is_contiguous():
+        raise KernelError("add_twin_rmsnorm: one tensor and one PartialSums at most, two norms at most, x contiguous")
+    if y:
+        _dev(y[0], "delta", out_dtype, 2)
+        if y[0].shape != x.shape or not y[0].is_contiguous():
+            raise KernelError(f"add_twin_rmsnorm: delta {tuple(y[0].shape)} does not match x {tuple(x.shape)}")
+    if parts and (tuple(parts[0].shape) != (T, D) or not parts[0].slabs.is_contiguous()):
+        raise KernelError(f"add_twin_rmsnorm: partial sums {tuple(parts[0].shape)} do not match x {tuple(x.shape)}")
+    for w, _ in norms:
+        _dev(w, "weight", torch.float32, 1)
+        if w.numel() != D or not w.is_contiguous():
+            raise KernelError(f"add_twin_rmsnorm: a norm's weight must hold {D} values")
+    outs = [torch.empty((T, D), dtype=out_dtype, device=x.device) for _ in norms]
+    if T:
+        args = []
+        for k in range(2):
+            args += [norms[k][0].data_ptr(), float(norms[k][1]), outs[k].data_ptr()] if k < len(norms) else [None, 0.0, None]
+        _check(_fn("twin_norm", "bn_twin_norm")(_code(out_dtype), x.data_ptr(), y[0].data_ptr() if y else None,
+                                                parts[0].slabs.data_ptr() if parts else None,
+                                                parts[0].slabs.shape[0] if parts else 0, *args, T, D, _stream()), "add_twin_rmsnorm")
+    return outs
 
 
 # --------------------------------------------------------------------------------------
@@ -2428,12 +2534,14 @@ MOE_SCORINGS = {"sigmoid": _build.header_constant("MOE_SCORE_SIGMOID", "moe.hip"
 
 def moe_route(h: torch.Tensor, router: torch.Tensor, top_k: int, scoring: str = "sigmoid", renormalize: bool = False, *,
               choice_bias: Optional[torch.Tensor] = None, weight_floor: float = 0.0, weight_scale: float = 1.0,
-              gate: Optional[torch.Tensor] = None, logit_bias: Optional[torch.Tensor] = None):
+              gate: Optional[torch.Tensor] = None, logit_bias: Optional[torch.Tensor] = None, groups=None):
     """(ids [T, top_k] int32, weights [T, top_k] float32): router logits z = router . h (+ logit_bias [E] float32) in
     float32 (router [E, D] float32, h in the activations' type), scores sigmoid(z) or softmax(z) over the experts, the top_k largest in
     descending order (ties: the lower index); renormalize divides the chosen scores by their sum (+ weight_floor);
     weight_scale multiplies the weights.  choice_bias [E] float32: the experts are chosen by score + bias, the weights
-    stay the plain scores.  gate [D] float32: a third result [T] float32, sigmoid(gate . h), a shared expert's gate."""
+    stay the plain scores.  gate [D] float32: a third result [T] float32, sigmoid(gate . h), a shared expert's gate.
+    groups = (count, keep): the experts form `count` equal groups of neighbours, a group ranks by its best member, and only
+    members of the best `keep` groups can be chosen."""
     require_gpu()
     _dev(h, "h", dims=2)
     _dev(router, "router", torch.float32, 2)
@@ -2449,6 +2557,9 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top_k: int, scoring: str = 
             _dev(t, nm, torch.float32, 1)
             if t.numel() != n or not t.is_contiguous():
                 raise KernelError(f"moe_route: {nm} must hold {n} float32 values")
+    n_groups, keep = (int(g) for g in groups) if groups is not None else (1, 1)
+    if n_groups < 1 or E % n_groups or not 1 <= keep <= n_groups or keep * (E // n_groups) < top_k:
+        raise KernelError(f"moe_route: the best {keep} of {n_groups} groups of {E} experts do not hold the {top_k} to be chosen")
     if not weight_floor >= 0.0:
         raise KernelError(f"moe_route: weight_floor {weight_floor} must not be negative")
     ids = torch.empty((T, top_k), dtype=torch.int32, device=h.device)
@@ -2460,7 +2571,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top_k: int, scoring: str = 
                                           choice_bias.data_ptr() if choice_bias is not None else None, float(weight_floor),
                                           float(weight_scale), gate.data_ptr() if gate is not None else None,
                                           gate_out.data_ptr() if gate is not None else None,
-                                          logit_bias.data_ptr() if logit_bias is not None else None, _stream()), "moe_route")
+                                          logit_bias.data_ptr() if logit_bias is not None else None, n_groups, keep, _stream()),
+               "moe_route")
     return (ids, wts) if gate is None else (ids, wts, gate_out)
 
 
@@ -2515,7 +2627,7 @@ def moe_experts(h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, ids: 
     UNARY_ACTIVATIONS), or, with `gated`, w_down[e] unit(gate rows . x, up rows . x) (w_up [E, 2 F, D]: F gate rows, then F
     up rows): slab j of the result [top_k, T, D] (float32) holds every token's j-th choice, computed on w h
     (weight_on_input) or scaled by w afterwards.  The feed-forward's output is the sum of the slabs.  extra_slabs: that
-    many more slabs behind the experts', left for the caller to fill."""
+    many more slabs behind the experts', left for the caller to fill.  ids from E on are identity experts: w h."""
     require_gpu()
     _dev(h, "h", dims=2)
     _dev(w_up, "w_up", h.dtype, 3)
@@ -2536,7 +2648,7 @@ def moe_experts(h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, ids: 
         hidden = torch.empty((n * K, F), dtype=torch.float32, device=h.device)
         _check(_fn("moe", "bn_moe_experts")(_code(h.dtype), h.data_ptr() + t0 * ld * h.element_size(), ld, w_up.data_ptr(),
                                             w_down.data_ptr(), ids.data_ptr() + t0 * K * 4, wts.data_ptr() + t0 * K * 4,
-                                            y.data_ptr() + t0 * D * 4, hidden.data_ptr(), n, T, D, F, K,
+                                            y.data_ptr() + t0 * D * 4, hidden.data_ptr(), n, T, D, F, E, K,
                                             0 if gated is not None else UNARY_ACTIVATIONS[activation], int(bool(weight_on_input)),
                                             int(gated is not None), float(unit.limit), float(unit.slope), float(unit.shift),
                                             _stream()), "moe_experts")
@@ -2585,7 +2697,7 @@ def moe_experts_grouped(h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tenso
     xg = torch.empty((n, D), dtype=torch.bfloat16, device=h.device)
     hidden = torch.empty((n, 2 * F if gated is not None else F), dtype=torch.bfloat16, device=h.device)
     _check(_fn("moe", "bn_moe_group")(h.data_ptr(), ld, ids.data_ptr(), wts.data_ptr(), work.data_ptr(), row_scale.data_ptr(),
-                                      xg.data_ptr(), T, D, E, K, MOE_TILE_ROWS, int(bool(weight_on_input)), _stream()),
+                                      xg.data_ptr(), T, D, E, K, MOE_TILE_ROWS, int(bool(weight_on_input)), y.data_ptr(), _stream()),
            "moe_group")
     row_map, tiles = work.data_ptr() + 4 * n, work.data_ptr() + 8 * n
     n_tiles = tiles + 12 * max_tiles

@@ -213,6 +213,14 @@ class PostNormedDelta:
         return ops.post_norm(x, self.delta, self.gain, self.alpha, self.norm.weight, self.norm.eps, **rows)
 
 
+class JoinedDelta:
+    """The outputs of a block's halves that read the same stream and join it together: tensors [T, D] in the activations'
+    type or ops.PartialSums."""
+
+    def __init__(self, deltas):
+        self.deltas = [d.compute() if isinstance(d, LazyDelta) else d for d in deltas]
+
+
 class ResidualStream:
     """The float32 residual stream of a step.  A part's output is held back as `pending` and
     is added by the kernel of the next norm, so the sum is formed once, in float32, without a
@@ -230,8 +238,8 @@ class ResidualStream:
         self.pending = delta
 
     def _pending_tensor(self):
-        if isinstance(self.pending, (NormedDelta, PostNormedDelta)):
-            raise TypeError("an output with a norm of its own is added by flush() or normed()")
+        if isinstance(self.pending, (NormedDelta, PostNormedDelta, JoinedDelta)):
+            raise TypeError("joined outputs and one with a norm of its own are added by flush() or normed()")
         if isinstance(self.pending, LazyDelta):
             self.pending = self.pending.compute()
         return self.pending
@@ -244,11 +252,48 @@ class ResidualStream:
         if isinstance(self.pending, PostNormedDelta):
             p, self.pending = self.pending, None
             p.apply(self.x)
+        if isinstance(self.pending, JoinedDelta):
+            self._join([], self._activations_type())
         if self.pending is not None:
             from .. import ops
             ops.residual_add(self.x, self._pending_tensor())
             self.pending = None
         return self.x
+
+    def _activations_type(self):
+        """The type of what is held back (partial sums are float32 whatever the activations are)."""
+        types = [d.dtype for d in self.pending.deltas if isinstance(d, torch.Tensor)]
+        return types[0] if types else torch.float32
+
+    def _join(self, norms, out_dtype) -> list:
+        """The new rows under each of the norms (two at most), after whatever is held back has joined the stream; one kernel
+        where it is a tensor, partial sums or one of each, and the norms are RMSNorms."""
+        from .. import ops
+        p = self.pending
+        deltas = p.deltas if isinstance(p, JoinedDelta) else [] if p is None else [p]
+        tensors = [d for d in deltas if isinstance(d, torch.Tensor)]
+        fits = (len(tensors) <= 1 and len(deltas) - len(tensors) <= 1 and self.x.is_contiguous()
+                and all(isinstance(d, (torch.Tensor, ops.PartialSums)) for d in deltas)
+                and all(d.dtype == out_dtype and d.is_contiguous() for d in tensors))
+        if not fits:
+            self.pending = None
+            if isinstance(p, JoinedDelta):
+                for d in p.deltas:
+                    self.add(d)
+            else:
+                self.pending = p
+            self.flush()
+            deltas = []
+        self.pending = None
+        if all(getattr(n, "normed_delta", False) for n in norms):
+            return ops.add_twin_rmsnorm(self.x, deltas, [(n.weight, n.eps) for n in norms], out_dtype) if deltas or norms else []
+        if deltas:
+            ops.add_twin_rmsnorm(self.x, deltas, [], out_dtype)
+        return [n.apply(self.x, None, out_dtype) for n in norms]
+
+    def normed_twice(self, norm_a, norm_b, out_dtype):
+        """The stream under two norms, for two parts that read the same rows."""
+        return tuple(self._join([norm_a, norm_b], out_dtype))
 
     def mixed_with_previous(self, mu: torch.Tensor, state: torch.Tensor, ctx) -> torch.Tensor:
         """x + (x' - x) * mu in the activations' type, x' the previous token's row of the stream as it stands here (zeros in
@@ -269,6 +314,10 @@ class ResidualStream:
         folded around, the result is an ops.DeferredNorm instead of a tensor.  With more rows than the fused
         products take, a consumer that has a method wants_deferred_norm(ctx, rows) is asked first (ctx: the step's
         context): one that would only apply the norm the plain way gets the plain norm, in one kernel instead of two."""
+        if isinstance(self.pending, JoinedDelta):
+            if rows is None:
+                return self._join([norm], out_dtype)[0]
+            self.flush()
         if isinstance(self.pending, PostNormedDelta):
             if rows is None and getattr(norm, "passes_rows", False):
                 p, self.pending = self.pending, None

@@ -7,6 +7,9 @@ With output norms (mixer_out_norm, ffn_out_norm) a half's output goes through a 
 stream: x += norm_out(mixer(norm(x))).  The stream holds such an output back with its norm (NormedDelta), and the
 kernel of the next norm forms the normed output, the sum and the next half's input in one pass.
 
+"parallel_prenorm": x += mixer(norm_1(x)) + ffn(norm_2(x)) -- both halves read the same stream, each under a norm of its own,
+and their outputs join it together; without a feed-forward the mixer's half alone.
+
 "postnorm": x <- norm(alpha x + gain mixer(x)); x <- norm(alpha x + gain ffn(x)) -- the norms stand behind the sums and
 their output is the stream; the halves read the stream itself.  alpha is a constant; with layer_scale every half's output
 has weights of its own (gain, one number per column); with token_shift the mixer reads the stream mixed with the previous
@@ -17,8 +20,8 @@ from dataclasses import replace
 
 import torch
 
-from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, CacheNeed, LazyDelta, NormedDelta, ParamSpec, Part, PartSpec,
-                   PostNormedDelta, StateNeed)
+from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, CacheNeed, JoinedDelta, LazyDelta, NormedDelta, ParamSpec, Part,
+                   PartSpec, PostNormedDelta, StateNeed)
 from .linear import upload
 from .shift import TokenShift
 
@@ -89,6 +92,31 @@ class PreNormBlock(Part):
             stream.add(self.ffn.forward(h, ctx, lazy_ok=True))
         else:
             stream.add(self.ffn.forward(h, ctx))
+        if tap is not None:
+            tap("layer_out", ctx.entry, stream, ctx)
+
+
+@BLOCKS.register("parallel_prenorm")
+class ParallelPreNormBlock(PreNormBlock):
+    """The tensors and children of a pre-norm block; one kernel adds the last block's outputs and forms both norms."""
+
+    def __init__(self, mixer: PartSpec, ffn: PartSpec | None, mixer_norm: PartSpec, ffn_norm: PartSpec | None = None):
+        super().__init__(mixer, ffn, mixer_norm, ffn_norm)
+
+    @staticmethod
+    def _run(part, *args):
+        return part.forward(*args, lazy_ok=True) if getattr(part, "gives_lazy_delta", False) else part.forward(*args)
+
+    def forward(self, stream, ctx, kv):
+        tap = getattr(ctx, "tap", None)        # diagnostics; both halves read the stream of "layer_in"
+        if tap is not None:
+            tap("layer_in", ctx.entry, stream, ctx)
+            tap("ffn_in", ctx.entry, stream, ctx)
+        if self.ffn is None:
+            stream.add(JoinedDelta([self._run(self.mixer, stream.normed(self.mixer_norm, ctx.act_dtype), ctx, kv)]))
+        else:
+            h_mixer, h_ffn = stream.normed_twice(self.mixer_norm, self.ffn_norm, ctx.act_dtype)
+            stream.add(JoinedDelta([self._run(self.mixer, h_mixer, ctx, kv), self._run(self.ffn, h_ffn, ctx)]))
         if tap is not None:
             tap("layer_out", ctx.entry, stream, ctx)
 

@@ -21,9 +21,15 @@ Options, each off by default:
   rot_dim     every query head is [head_dim plain, rot_dim rotated] and W_dkv h has rot_dim more rows behind the latent's: one
               rotated key part that all heads share, not normed.  The score is (q_plain . k_plain + q_rot . k_rot) * scale.  The
               rotation turns dimension i with dimension i + rot_dim / 2 by position * f_i (rot_theta, rot_scaling as
-              parts/position.py's; a "yarn" scaling also multiplies cosine and sine).  The cache's key row is then
+              parts/position.py's; a "yarn" scaling also multiplies cosine and sine), or, rot_interleaved, dimension 2i with
+              2i + 1.  The cache's key row is then
               [c, k_rot] (kv_rank + rot_dim wide) and the query in the latent's space [W_uk^T q_plain, q_rot]; values stay c.
   gate        "head": one gate number per head, sigmoid(W_g h)_i multiplies head i's output (wg [heads, hidden])
+  sink        every head's softmax has one more term without a value: exp(sink_i) joins its denominator (tensor sink
+              [heads], not scaled)
+
+The stored rows may be a little wider than their numbers, zeros behind them (ops.latent_row_widths), so that the
+matrix-core kernels take sizes between theirs; W_uk's and W_uv's rearranged copies hold zeros there.
 
 own_latent False: the layer has no W_dkv; its schedule entry reads the cache of the entry that has (ScheduleEntry.kv_from),
 with its own W_uk and W_uv, queries, gate and output projection.
@@ -44,7 +50,7 @@ class LatentAttention(Part):
 
     def __init__(self, hidden: int, n_heads: int, head_dim: int, kv_rank: int, scale: float, eps: float,
                  v_head_dim: int = 0, own_latent: bool = True, gate=True, q_rank: int = 0, rot_dim: int = 0,
-                 rot_theta: float = 10000.0, rot_scaling=None):
+                 rot_theta: float = 10000.0, rot_scaling=None, rot_interleaved: bool = False, sink: bool = False):
         self.hidden, self.H, self.hs, self.rank = int(hidden), int(n_heads), int(head_dim), int(kv_rank)
         self.vd = int(v_head_dim) or self.hs
         if gate not in (False, True, "head"):
@@ -54,11 +60,13 @@ class LatentAttention(Part):
         self.q_rank, self.rot = int(q_rank), int(rot_dim)
         if self.rot % 2 or self.rot < 0 or self.q_rank < 0:
             raise ValueError(f"latent attention: rot_dim {rot_dim} must be even and q_rank {q_rank} not negative")
-        self.kw = self.rank + self.rot               # width of a cached key row: the latent, then the rotated part
-        if self.rank % 2 or self.rank < 2 or self.kw > ops.MAX_HEAD_DIM:
+        if self.rank % 2 or self.rank < 2 or self.rank + self.rot > ops.MAX_LATENT_KEY or self.rank > ops.MAX_LATENT_VALUE:
             raise ValueError(f"latent attention: kv_rank {self.rank} (+ rot_dim {self.rot}) is not supported by the attention "
-                             f"kernels (even, at most {ops.MAX_HEAD_DIM})")
-        if max(self.hs + self.rot, self.rank) > ops.HEAD_LINEAR_MAX_IN:
+                             f"kernels (even, at most {ops.MAX_LATENT_VALUE}, {ops.MAX_LATENT_KEY} together)")
+        # widths of a cached key row (the latent, then the rotated part) and of a value row (the latent)
+        self.kw, self.vw = ops.latent_row_widths(self.rank, self.rot)
+        self.interleaved, self.has_sink, self.sink = bool(rot_interleaved), bool(sink), None
+        if max(self.hs + self.rot, self.vw) > ops.HEAD_LINEAR_MAX_IN:
             raise ValueError(f"latent attention: head_dim {self.hs} / kv_rank {self.rank} above {ops.HEAD_LINEAR_MAX_IN}")
         self.rot_scaling = dict(rot_scaling) if rot_scaling else None
         self.rot_mult = rope_magnitude(self.rot_scaling)
@@ -66,7 +74,7 @@ class LatentAttention(Part):
         self.inv_freq = self.dq_norm = None
         self.uq = Linear()                          # W_uq when the queries have a latent of their own
         self.proj, self.o = Linear(), Linear()      # proj: [W_q (or W_dq); W_g; W_dkv] stacked, one product
-        self.uk = self.uv_t = self.dkv_norm = None   # [H, head_dim, rank] and [H, rank, v_head_dim]: both [head, in, out]
+        self.uk = self.uv_t = self.dkv_norm = None   # [H, head_dim + rot, kw] and [H, vw, v_head_dim]: both [head, in, out]
 
     @property
     def q_dim(self):
@@ -91,8 +99,10 @@ class LatentAttention(Part):
                   "wo": ParamSpec((D, self.o_dim))})
         if self.gated:
             t["wg"] = ParamSpec((self.g_dim, D))
+        if self.has_sink:
+            t["sink"] = ParamSpec((self.H,), "normal")
         if self.own:
-            t.update({"wdkv": ParamSpec((self.kw, D)), "dkv_norm": ParamSpec((self.rank,), "ones")})
+            t.update({"wdkv": ParamSpec((self.rank + self.rot, D)), "dkv_norm": ParamSpec((self.rank,), "ones")})
         return t
 
     def load(self, tensors, device, dtype):
@@ -107,16 +117,25 @@ class LatentAttention(Part):
         # W_uk of head i is [head_dim, rank]: already [in, out] for q' = W_uk^T q; W_uv of head i is [v_head_dim, rank]:
         # turned once to [rank, v_head_dim].  With a rotated part a head's matrix gets rot_dim more rows and columns that
         # hand the rotated query dimensions on as they are (an identity block), so one product per head makes the whole
-        # query of the latent's space.
+        # query of the latent's space.  Columns and rows that only fill a stored row up are zero.
         uk = upload(tensors["wuk"], device, dtype).reshape(self.H, self.hs, self.rank)
-        if self.rot:
+        if self.kw != self.rank:
             full = torch.zeros((self.H, self.hs + self.rot, self.kw), dtype=dtype, device=uk.device)
             full[:, :self.hs, :self.rank] = uk
-            full[:, self.hs:, self.rank:] = torch.eye(self.rot, dtype=dtype, device=uk.device)
+            if self.rot:
+                full[:, self.hs:, self.rank:self.rank + self.rot] = torch.eye(self.rot, dtype=dtype, device=uk.device)
             uk = full
+        if self.rot:
             self.inv_freq = self._freq_host.to(device).contiguous()
         self.uk = uk.contiguous()
-        self.uv_t = upload(tensors["wuv"], device, dtype).reshape(self.H, self.vd, self.rank).transpose(1, 2).contiguous()
+        uv = upload(tensors["wuv"], device, dtype).reshape(self.H, self.vd, self.rank).transpose(1, 2)
+        if self.vw != self.rank:
+            full = torch.zeros((self.H, self.vw, self.vd), dtype=dtype, device=uv.device)
+            full[:, :self.rank] = uv
+            uv = full
+        self.uv_t = uv.contiguous()
+        if self.has_sink:
+            self.sink = upload(tensors["sink"], device, torch.float32)
         if self.own:
             self.dkv_norm = upload(tensors["dkv_norm"], device, torch.float32)
 
@@ -124,46 +143,48 @@ class LatentAttention(Part):
         return [self.proj, self.o] + ([self.uq] if self.q_rank else [])
 
     def cache_need(self) -> CacheNeed:
-        return CacheNeed(kv=KVNeed(1, self.kw, 0, v_head_dim=self.rank, v_layout="transposed"))
+        return CacheNeed(kv=KVNeed(1, self.kw, 0, v_head_dim=self.vw, v_layout="transposed"))
 
     def forward(self, h, ctx, kv):
-        H, hs, vd, R = self.H, self.hs, self.vd, self.rank
+        H, R, KW, VW = self.H, self.rank, self.kw, self.vw
         if isinstance(h, ops.DeferredNorm):
             h = h.materialize()
         if kv.writes != self.own:
             raise ValueError("latent attention: a layer with a down-projection writes its own cache, one without reads another's")
         p = self.proj(h)                                    # [T, q columns (+ gate columns) (+ R + rot)]
         q_cols = self.q_rank or self.q_dim
-        if self.own:
-            ops.latent_store(p, q_cols + self.g_dim, R, self.dkv_norm, self.eps, ctx.positions,
-                             ctx.seq_index, kv.block_table, kv.k_pages, kv.v_pages, rot_dims=self.rot, inv_freq=self.inv_freq,
-                             rot_mult=self.rot_mult)
+        cq = None
+        if self.own:                                         # with the queries' own latent normed in the same kernel
+            cq = ops.latent_store(p, q_cols + self.g_dim, R, self.dkv_norm, self.eps, ctx.positions,
+                                  ctx.seq_index, kv.block_table, kv.k_pages, kv.v_pages, rot_dims=self.rot, inv_freq=self.inv_freq,
+                                  rot_mult=self.rot_mult, interleaved=self.interleaved, row_widths=(KW, VW),
+                                  query=(0, self.dq_norm) if self.q_rank else None)
         if self.q_rank:
-            cq = p[:, :q_cols].contiguous() if p.shape[1] != q_cols else p
-            qh = self.uq(ops.rmsnorm_mean(cq, self.dq_norm, None, None, self.eps))       # [T, H (hs + rot)]
+            if cq is None:
+                cq = ops.rmsnorm_mean(p[:, :q_cols].contiguous(), self.dq_norm, None, None, self.eps)
+            qh = self.uq(cq)                                 # [T, H (hs + rot)]
         else:
             qh = p[:, :q_cols]
-        KW = self.kw
-        q = ops.head_linear(qh, self.uk)                     # [T, H KW]: the queries in the latent's space
-        if self.rot:
-            ops.rope_heads(q, ctx.positions, self.inv_freq, H, KW, R, self.rot, self.rot_mult)
-        out = torch.empty((h.shape[0], H * R), dtype=h.dtype, device=h.device)
-        on_matrix_cores = ops.attention_general_supported(h.dtype, KW, R) and ops.GENERAL_PROMPT_ON_MATRIX_CORES
+        rotate = (ctx.positions, self.inv_freq, R, self.rot_mult, self.interleaved) if self.rot else None
+        q = ops.head_linear(qh, self.uk, rotate=rotate)      # [T, H KW]: the queries in the latent's space
+        out = torch.empty((h.shape[0], H * VW), dtype=h.dtype, device=h.device)
+        on_matrix_cores = ops.attention_general_supported(h.dtype, KW, VW) and ops.GENERAL_PROMPT_ON_MATRIX_CORES
         if ctx.is_decode and on_matrix_cores:
             n_splits, chunk, _ = ops.general_decode_plan(ctx.n_rows, H, 1, kv.max_len)
-            ops.attention_general_decode(q, out, kv.k_pages, kv.v_pages, kv.block_table, ctx.seq_lens, H, 1, KW, R, self.scale,
-                                         n_splits=n_splits, chunk=chunk, max_len_dev=ctx.max_len_dev if n_splits > 1 else None)
+            ops.attention_general_decode(q, out, kv.k_pages, kv.v_pages, kv.block_table, ctx.seq_lens, H, 1, KW, VW, self.scale,
+                                         n_splits=n_splits, chunk=chunk, max_len_dev=ctx.max_len_dev if n_splits > 1 else None,
+                                         sink=self.sink)
         elif ctx.is_decode:
             n_splits, chunk = ops.decode_splits(ctx.n_rows, H, 1, kv.max_len, h.dtype, target_wgs=ops.VECTOR_DECODE_TARGET_WGS)
             ops.attention(q, out, kv.k_pages, kv.v_pages, kv.block_table, H, 1, KW, self.scale, seq_lens=ctx.seq_lens,
                           n_splits=n_splits, chunk=chunk, max_len_dev=ctx.max_len_dev if n_splits > 1 else None,
-                          v_transposed=True, blocked=False, v_dim=R)
+                          v_transposed=True, blocked=False, v_dim=VW, sink=self.sink)
         elif on_matrix_cores:
-            ops.attention_general_prompt(q, out, kv.k_pages, kv.v_pages, kv.block_table, H, 1, KW, R, self.scale,
-                                         ctx.tiles(ops.GENERAL_PROMPT_TILE))
+            ops.attention_general_prompt(q, out, kv.k_pages, kv.v_pages, kv.block_table, H, 1, KW, VW, self.scale,
+                                         ctx.tiles(ops.GENERAL_PROMPT_TILE), sink=self.sink)
         else:
             _, _, qt = ops.attention_row_shape(H, 1, False)
             ops.attention(q, out, kv.k_pages, kv.v_pages, kv.block_table, H, 1, KW, self.scale, tiles=ctx.tiles(qt), qt=qt,
-                          v_transposed=True, blocked=False, v_dim=R)
+                          v_transposed=True, blocked=False, v_dim=VW, sink=self.sink)
         gate = p[:, q_cols:q_cols + self.g_dim] if self.gated else None
         return self.o(ops.head_linear(out, self.uv_t, gate, gate_per_head=self.gate_per_head))

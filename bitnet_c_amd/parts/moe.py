@@ -17,6 +17,10 @@ Options beside that form, each off by default:
   gated            (without expert_limit) the experts are plain gated units W_down,e (act(W_gate,e x) * (W_up,e x)) with
                    act = silu: the unit above without bounds, slope 1 and shift 0
   router_bias      a tensor `router_bias` [n_experts] added to the logits themselves, before scoring and choice
+  identity_experts that many more rows of the router (and entries of correction and router_bias) behind the experts': experts
+                   without tensors whose output is the feed-forward's input itself, chosen and weighted like any other
+  groups (count, keep)   the experts (identity experts included) form `count` equal groups of neighbours; a group ranks by its
+                   best member's choice score, and only members of the best `keep` groups can be chosen
   shared_intermediate (with shared_limit)   one more gated unit of that width that every token runs (shared.w_gate,
                    shared.w_up, shared.w_down), its output times sigmoid(shared.gate . h), one number per token
 
@@ -44,7 +48,7 @@ class MoEFFN(Part):
                  scoring: str = "sigmoid", renormalize: bool = False, weight_on: str = "input", expert_limit: float = 0.0,
                  gate_slope: float = 1.702, up_shift: float = 1.0, choice_bias: bool = False, weight_floor: float = 0.0,
                  weight_scale: float = 1.0, shared_intermediate: int = 0, shared_limit: float = 0.0, gated: bool = False,
-                 router_bias: bool = False):
+                 router_bias: bool = False, identity_experts: int = 0, groups=None):
         if activation not in ops.UNARY_ACTIVATIONS:
             raise ValueError(f"moe: unknown activation {activation!r}; known: {sorted(ops.UNARY_ACTIVATIONS)}")
         if scoring not in ops.MOE_SCORINGS:
@@ -52,8 +56,15 @@ class MoEFFN(Part):
         if weight_on not in ("input", "output"):
             raise ValueError(f"moe: weight_on {weight_on!r} is neither 'input' nor 'output'")
         self.hidden, self.E, self.K, self.F = int(hidden), int(n_experts), int(top_k), int(intermediate)
-        if not 1 <= self.K <= self.E or self.E > ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"moe: top_k {self.K} of {self.E} experts (at most {ops.MOE_MAX_EXPERTS})")
+        self.n_identity = int(identity_experts)
+        self.R = self.E + self.n_identity                    # rows of the router
+        if self.E < 1 or self.n_identity < 0 or not 1 <= self.K <= self.R or self.R > ops.MOE_MAX_EXPERTS:
+            raise ValueError(f"moe: top_k {self.K} of {self.E} experts and {self.n_identity} identity experts (at most "
+                             f"{ops.MOE_MAX_EXPERTS})")
+        self.groups = tuple(int(g) for g in groups) if groups is not None else (1, 1)
+        count, keep = self.groups
+        if count < 1 or self.R % count or not 1 <= keep <= count or keep * (self.R // count) < self.K:
+            raise ValueError(f"moe: the best {keep} of {count} groups of {self.R} experts do not hold the {self.K} to be chosen")
         self.activation, self.scoring, self.renormalize = activation, scoring, bool(renormalize)
         self.weight_on_input = weight_on == "input"
         self.unit = ops.ClampedUnit(float(expert_limit), float(gate_slope), float(up_shift)) if expert_limit else None
@@ -73,11 +84,11 @@ class MoEFFN(Part):
         self.router = self.w_up = self.w_down = self.choice_bias = self.shared_gate = self.router_bias = None
 
     def tensors(self):
-        t = {"router": ParamSpec((self.E, self.hidden))}
+        t = {"router": ParamSpec((self.R, self.hidden))}
         if self.has_choice_bias:
-            t["correction"] = ParamSpec((self.E,), "normal")
+            t["correction"] = ParamSpec((self.R,), "normal")
         if self.has_router_bias:
-            t["router_bias"] = ParamSpec((self.E,), "normal")
+            t["router_bias"] = ParamSpec((self.R,), "normal")
         for e in range(self.E):
             if self.unit is not None:
                 t[f"e{e}.w_gate"] = ParamSpec((self.F, self.hidden))
@@ -116,7 +127,7 @@ class MoEFFN(Part):
             h = h.materialize()
         routed = ops.moe_route(h, self.router, self.K, self.scoring, self.renormalize, choice_bias=self.choice_bias,
                                weight_floor=self.weight_floor, weight_scale=self.weight_scale, gate=self.shared_gate,
-                               logit_bias=self.router_bias)
+                               logit_bias=self.router_bias, groups=self.groups)
         ids, wts = routed[0], routed[1]
         experts = ops.moe_experts_grouped if ops.moe_grouped_supported(h.shape[0], self.hidden, self.F, h.dtype) else ops.moe_experts
         y = experts(h, self.w_up, self.w_down, ids, wts, self.activation, self.weight_on_input, gated=self.unit,

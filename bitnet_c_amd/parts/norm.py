@@ -3,6 +3,7 @@
 type; the weight is kept in float32.  `scalar`: the model folder holds one number for all
 coordinates (a tensor without dimensions); it is spread over the coordinates at load, and
 every kernel that takes this norm, folded into a product or not, sees a weight vector.
+`offset`: the stored weight w means offset + w (1: a weight stored around zero); the sum is formed once, at load, in float32.
 
 "none": no norm at all: the part behind it reads the stream itself, in the activations' type (a block whose norms sit on
 its parts' outputs only)."""
@@ -22,15 +23,17 @@ class RMSNorm(Part):
     takes_partial_sums = True    # apply() accepts ops.PartialSums as the delta
     normed_delta = True          # weight and eps are all that ops.add_normed_rmsnorm needs: it may be a block's output norm
 
-    def __init__(self, dim: int, eps: float, scalar: bool = False):
-        self.dim, self.eps, self.scalar = int(dim), float(eps), bool(scalar)
+    def __init__(self, dim: int, eps: float, scalar: bool = False, offset: float = 0.0):
+        self.dim, self.eps, self.scalar, self.offset = int(dim), float(eps), bool(scalar), float(offset)
         self.weight = None
 
     def tensors(self):
-        return {"weight": ParamSpec(() if self.scalar else (self.dim,), init="ones")}
+        return {"weight": ParamSpec(() if self.scalar else (self.dim,), init="zeros" if self.offset == 1.0 else "ones")}
 
     def load(self, tensors, device, dtype):
         w = upload(tensors["weight"], device, torch.float32)
+        if self.offset:
+            w = w + self.offset
         self.weight = w.reshape(1).expand(self.dim).contiguous() if self.scalar else w
 
     def apply(self, x, delta, out_dtype, rows=None):

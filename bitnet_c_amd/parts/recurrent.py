@@ -21,6 +21,11 @@ input (zero before the first token; the last h of a step is part of the state):
     q, k = silu(W_q h), silu(W_k h)   heads x head_dim;   v = silu(W_v h)   heads x v_head_dim
     S <- decay_head S + k_t v_t^T;    o_t = S^T q_t                       no other scale
     y = W_o (o / rms_row(o) * norm * sigmoid(W_g h))                     the heads' outputs normed together, eps inside the root
+
+"retention": the same recurrence over rotated queries and keys (csrc/lightning.hip with another feed):
+    q, k = rot_p(W_q h), rot_p(W_k h) / sqrt(head_dim)    heads x head_dim;   v = W_v h    heads x v_head_dim
+    S <- decay_head S + k_t v_t^T;    o_t = S^T q_t
+    y = W_o (o / rms_head(o) * silu(W_g h))               every head divided by its own root mean square, no weight
 """
 from __future__ import annotations
 
@@ -29,6 +34,7 @@ import torch
 from .. import ops
 from .base import MIXERS, CacheNeed, ParamSpec, Part, StateNeed
 from .linear import Linear, upload
+from .position import rope_frequencies
 
 
 def _sequences(ctx):
@@ -132,24 +138,21 @@ class MinGRU(Part):
         return self.o(y)
 
 
-@MIXERS.register("lightning")
-class Lightning(Part):
+class DecayedSums(Part):
+    """What linear attention with a constant decay per head shares: the four projections stacked, the decays, the state."""
     prompt_capturable = True    # a prompt step is read from the context's device tensors alone
+    what = "decayed sums"
 
-    def __init__(self, hidden: int, n_heads: int, head_dim: int, decay, eps: float, v_head_dim: int = 0,
-                 gate_activation: str = "sigmoid"):
+    def __init__(self, hidden: int, n_heads: int, head_dim: int, decay, eps: float, v_head_dim: int = 0):
         self.hidden, self.H, self.hs, self.eps = int(hidden), int(n_heads), int(head_dim), float(eps)
         self.vd = int(v_head_dim) or self.hs
         self.decay_values = tuple(float(d) for d in decay)
         if len(self.decay_values) != self.H or not all(0.0 <= d <= 1.0 for d in self.decay_values):
-            raise ValueError(f"lightning: one decay in [0, 1] per head, got {len(self.decay_values)} for {self.H} heads")
+            raise ValueError(f"{self.what}: one decay in [0, 1] per head, got {len(self.decay_values)} for {self.H} heads")
         if not ops.lightning_supported(self.hs, self.vd):
-            raise ValueError(f"lightning: head_dim {self.hs} is not supported by the kernel (at most {ops.LIGHTNING_MAX_DIM})")
-        if gate_activation not in ops.UNARY_ACTIVATIONS:
-            raise ValueError(f"lightning: unknown gate activation {gate_activation!r}; known: {sorted(ops.UNARY_ACTIVATIONS)}")
-        self.gate_activation = gate_activation
+            raise ValueError(f"{self.what}: head_dim {self.hs} is not supported by the kernel (at most {ops.LIGHTNING_MAX_DIM})")
         self.qkvg, self.o = Linear(), Linear()        # the four projections stacked: one product
-        self.decay = self.norm = None
+        self.decay = None
 
     @property
     def k_col(self):
@@ -166,13 +169,12 @@ class Lightning(Part):
     def tensors(self):
         D, A, B = self.hidden, self.H * self.hs, self.H * self.vd
         return {"wq": ParamSpec((A, D)), "wk": ParamSpec((A, D)), "wv": ParamSpec((B, D)), "wg": ParamSpec((B, D)),
-                "norm": ParamSpec((B,), "ones"), "wo": ParamSpec((D, B))}
+                "wo": ParamSpec((D, B))}
 
     def load(self, tensors, device, dtype):
         w = torch.cat([upload(tensors[n], device, dtype) for n in ("wq", "wk", "wv", "wg")], dim=0).contiguous()
         self.qkvg.load(w, None, device, dtype)
         self.o.load(tensors["wo"], None, device, dtype)
-        self.norm = upload(tensors["norm"], device, torch.float32)
         self.decay = torch.tensor(self.decay_values, dtype=torch.float64).to(torch.float32).to(device)
 
     def linears(self):
@@ -182,11 +184,62 @@ class Lightning(Part):
         # per head a [head_dim, v_head_dim] matrix, float32
         return CacheNeed(state=StateNeed((self.H * self.hs * self.vd,), torch.float32, device_addressed=True))
 
+
+@MIXERS.register("lightning")
+class Lightning(DecayedSums):
+    what = "lightning"
+
+    def __init__(self, hidden: int, n_heads: int, head_dim: int, decay, eps: float, v_head_dim: int = 0,
+                 gate_activation: str = "sigmoid"):
+        super().__init__(hidden, n_heads, head_dim, decay, eps, v_head_dim)
+        if gate_activation not in ops.UNARY_ACTIVATIONS:
+            raise ValueError(f"lightning: unknown gate activation {gate_activation!r}; known: {sorted(ops.UNARY_ACTIVATIONS)}")
+        self.gate_activation = gate_activation
+        self.norm = None
+
+    def tensors(self):
+        t = super().tensors()
+        wo = t.pop("wo")
+        return dict(t, norm=ParamSpec((self.H * self.vd,), "ones"), wo=wo)
+
+    def load(self, tensors, device, dtype):
+        super().load(tensors, device, dtype)
+        self.norm = upload(tensors["norm"], device, torch.float32)
+
     def forward(self, h, ctx, kv):
         x = self.qkvg(h)
         o = ops.lightning_scan(x, 0, self.k_col, self.v_col, self.decay, kv.state, ctx.slot_ids, self.H, self.hs, self.vd,
                                **_sequences(ctx))
         y = ops.row_norm_gate(o, x[:, self.g_col:], self.norm, self.eps, self.gate_activation)
+        return self.o(y)
+
+
+@MIXERS.register("retention")
+class Retention(DecayedSums):
+    """rope_dims (even, at most head_dim; 0: no rotation) dimensions of every query and key head turn in split-half pairs,
+    dimension i by position * rope_theta^(-2i / rope_dims)."""
+    what = "retention"
+
+    def __init__(self, hidden: int, n_heads: int, head_dim: int, decay, eps: float, v_head_dim: int = 0, rope_dims: int = 0,
+                 rope_theta: float = 10000.0):
+        super().__init__(hidden, n_heads, head_dim, decay, eps, v_head_dim)
+        self.rope_dims = int(rope_dims)
+        if self.rope_dims % 2 or not 0 <= self.rope_dims <= self.hs:
+            raise ValueError(f"retention: rope_dims {rope_dims} must be even and at most head_dim {self.hs}")
+        self._freq_host = rope_frequencies(self.rope_dims, float(rope_theta)) if self.rope_dims else None
+        self.inv_freq = None
+
+    def load(self, tensors, device, dtype):
+        super().load(tensors, device, dtype)
+        if self.rope_dims:
+            self.inv_freq = self._freq_host.to(device).contiguous()
+
+    def forward(self, h, ctx, kv):
+        x = self.qkvg(h)
+        o = ops.lightning_scan(x, 0, self.k_col, self.v_col, self.decay, kv.state, ctx.slot_ids, self.H, self.hs, self.vd,
+                               silu=False, inv_freq=self.inv_freq, positions=ctx.positions if self.rope_dims else None,
+                               k_scale=self.hs ** -0.5, **_sequences(ctx))
+        y = ops.head_norm_gate(o, x[:, self.g_col:], None, self.H, self.vd, self.eps)
         return self.o(y)
 
 

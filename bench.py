@@ -280,10 +280,34 @@ def _pafutar_configs(z):
     return paf, faz, son, _llama_config(z)
 
 
+def _zenasun_configs(z):
+    """(Zenasun config.json, Mutirax config.json, Fazopel config.json, Llama config.json) of equal width, layer runs and
+    attention heads: two retention layers (heads as many and as wide as the attention's), then a latent attention layer with
+    Mutirax's latents, repeated; every layer chooses `top` of `experts` experts, an eighth of them identity experts, in the
+    best two of four groups; an expert's three matrices times `top` are as large as the gated feed-forward's."""
+    gated = _llama_config(z)["intermediate_size"]
+    H, identity = z["heads"], z["experts"] // 8
+    moe = dict(kind="moe", expert=dict(ff=gated // z["top"] // 64 * 64),
+               router=dict(experts=z["experts"] - identity, identity=identity, top=z["top"], groups=dict(count=4, keep=2)))
+    ret = dict(heads=H, dim=z["dim"], vdim=z["dim"], decay=[round(1.0 - 2.0 ** -(5.0 + 3.0 * h / max(H - 1, 1)), 9) for h in range(H)],
+               rot=dict(base=10000.0, dims=z["dim"]))
+    lat = dict(heads=H, dim=z["dim"], rot_dim=z["rot_dims"], vdim=z["dim"], kv_rank=256 - z["rot_dims"], q_rank=z["width"] // 2,
+               scale=(z["dim"] + z["rot_dims"]) ** -0.5, rot=dict(base=100000.0, dims=z["rot_dims"]))
+    layers = [dict(type="latent_attention", mixer=lat, mlp=moe) if i % 3 == 2 else dict(type="retention", mixer=ret, mlp=moe)
+              for i in range(z["layers"])]
+    zen = dict(architecture="Zenasun", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6), embedding=dict(scale=8.0),
+               logit_softcap=30.0, layers=layers)
+    mut, faz, _, llama = _mutirax_configs(z)
+    return zen, mut, faz, llama
+
+
 def _design_configs(design, z):
     """name -> config.json: the design, then what it is measured beside (the Llama-style decoder of equal width, layers,
     attention heads and (nearly) equal weight bytes read per token; for Fazopel also Sonodra, the closest of the others;
-    for Mutirax Fazopel and Sonodra; for Pafutar both, with its own kind of layer in every layer)."""
+    for Mutirax Fazopel and Sonodra; for Pafutar both, with its own kind of layer in every layer; for Zenasun Mutirax and
+    Fazopel)."""
+    if design == "zenasun":
+        return dict(zip(("zenasun", "mutirax", "fazopel", "llama"), _zenasun_configs(z)))
     if design == "pafutar":
         return dict(zip(("pafutar", "fazopel", "sonodra", "llama"), _pafutar_configs(z)))
     if design == "mutirax":
@@ -401,7 +425,7 @@ def main() -> int:
     ap.add_argument("--prompt-lens", default=None, metavar="LO,HI", help="prompt lengths of the decode batches")
     ap.add_argument("--prefill-tokens", type=int, default=PREFILL_TOKENS, help="tokens of the measured prompt step")
     ap.add_argument("--design-alone", action="store_true", help="with --design: the design alone, for profiling")
-    ap.add_argument("--design", choices=["sunusun", "sonodra", "fazopel", "mutirax", "pafutar"], default=None,
+    ap.add_argument("--design", choices=["sunusun", "sonodra", "fazopel", "mutirax", "pafutar", "zenasun"], default=None,
                     help="instead of the benchmark: prefill and decode of this design beside the Llama-style decoder of equal "
                          "width, heads, layers and weight bytes, at the sizes of --design-size (random weights; one JSON line)")
     ap.add_argument("--design-size", choices=sorted(DESIGN_SIZES), default="2048")

@@ -22,7 +22,6 @@
 #include <math.h>
 
 #define MOE_MAX_EXPERTS 1024
-#define MOE_PER_LANE (MOE_MAX_EXPERTS / BN_WAVE)
 #define MOE_SCORE_SIGMOID 0
 #define MOE_SCORE_SOFTMAX 1
 
@@ -31,7 +30,7 @@ struct RouteArgs {
     const float* wr;          // [E, D] float32
     int* ids;                 // [T, K]
     float* wts;               // [T, K]
-    int ld, D, E, K, scoring, renorm;
+    int ld, T, D, E, K, scoring, renorm;
     const float* bias;        // [E] added to the scores for the choice alone; null: the choice goes by the scores
     const float* zbias;       // [E] added to the logits themselves (a router with a bias); null: none
     const float* gate_w;      // [D]: gate_out[t] = sigmoid(gate_w . h); null: none
@@ -40,58 +39,103 @@ struct RouteArgs {
     int groups, keep;         // groups > 1: E / groups neighbours a group, the best `keep` groups stay in the choice
 };
 
-#define MOE_ROUTE_THREADS 256
+// A wave an expert as far as a workgroup's 16 waves go.  Steps of few rows (MOE_ROUTE_FEW_ROWS): a workgroup a token.  Steps
+// of many: four tokens a workgroup, whose rows lie in shared memory and whose waves read a router row once for all four and
+// then choose for a token each.  A token's sums have one order either way.
+#define MOE_ROUTE_FEW_ROWS 256
+#define MOE_ROUTE_THREADS 1024
+#define MOE_ROUTE_TOKENS 4
 
-// One workgroup a token: its waves take the experts in turn (a row of the router as 16-byte loads across the lanes, several
-// in flight), the first wave then chooses.
-template <typename T>
-__global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs a) {
-    extern __shared__ __align__(16) float hs[];          // the token's row as float32, then the experts' logits
-    float* zs = hs + ((a.D + 3) & ~3);
-    const int t = blockIdx.x, lane = threadIdx.x & (BN_WAVE - 1), wave = threadIdx.x / BN_WAVE;
-    const T* h = reinterpret_cast<const T*>(a.h) + (size_t)t * a.ld;
-    for (int d = threadIdx.x; d < a.D; d += MOE_ROUTE_THREADS) hs[d] = to_f32(h[d]);
-    __syncthreads();
+__device__ __forceinline__ float4 moe_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 moe_load4(const bf16* p) {
+    const uint2 t = *reinterpret_cast<const uint2*>(p);
+    return make_float4(bf16lo_to_f32(t.x), bf16hi_to_f32(t.x), bf16lo_to_f32(t.y), bf16hi_to_f32(t.y));
+}
+
+__host__ __device__ __forceinline__ int moe_route_row_bytes(int D, int elt) { return (D * elt + 15) & ~15; }
+
+// The waves take the experts in turn (a row of the router as 16-byte loads across the lanes with the tokens' rows beside it,
+// several in flight); then wave i chooses for token i.  PL: experts a lane of such a wave holds, E <= 64 PL; TK: tokens of the
+// workgroup, which has at least as many waves.
+template <typename T, int PL, int TK>
+__global__ __launch_bounds__(MOE_ROUTE_THREADS, PL == 1 ? 8 : 4) void moe_route_kernel(RouteArgs a) {
+    // the tokens' rows (TK > 1; whole 16-byte groups a row), then per token the experts' logits and the groups' best values
+    extern __shared__ __align__(16) unsigned char route_raw[];
+    const int t0 = blockIdx.x * TK, lane = threadIdx.x & (BN_WAVE - 1), wave = threadIdx.x / BN_WAVE;
+    const T* h[TK];
+#pragma unroll
+    for (int k = 0; k < TK; ++k) h[k] = reinterpret_cast<const T*>(a.h) + (size_t)min(t0 + k, a.T - 1) * a.ld;
+    const bool whole = a.D % 4 == 0 && (TK > 1 || (a.ld % 4 == 0 && ((uintptr_t)a.h & (4 * sizeof(T) - 1)) == 0));
+    const int row_bytes = TK > 1 ? moe_route_row_bytes(a.D, (int)sizeof(T)) : 0;
+    float* route_smem = reinterpret_cast<float*>(route_raw + TK * row_bytes);
+    if (TK > 1) {
+#pragma unroll
+        for (int k = 0; k < TK; ++k) {
+            T* hs = reinterpret_cast<T*>(route_raw + k * row_bytes);
+            if (a.ld * sizeof(T) % 16 == 0 && a.D * sizeof(T) % 16 == 0 && ((uintptr_t)a.h & 15) == 0) {
+                for (int d = threadIdx.x; d < (int)(a.D * sizeof(T) / 16); d += blockDim.x)
+                    reinterpret_cast<uint4*>(hs)[d] = reinterpret_cast<const uint4*>(h[k])[d];
+            } else {
+                for (int d = threadIdx.x; d < a.D; d += blockDim.x) hs[d] = h[k][d];
+            }
+            h[k] = hs;
+        }
+        __syncthreads();
+    }
     // the shared expert's gate is one more row: it takes its turn among the waves after the experts
-    for (int e = wave; e < a.E + (a.gate_w ? 1 : 0); e += MOE_ROUTE_THREADS / BN_WAVE) {
+    for (int e = wave; e < a.E + (a.gate_w ? 1 : 0); e += blockDim.x / BN_WAVE) {
         const float* w = e < a.E ? a.wr + (size_t)e * a.D : a.gate_w;
-        float s = 0.f;
-        if (a.D % 4 == 0) {
-#pragma unroll 4
+        float s[TK];
+#pragma unroll
+        for (int k = 0; k < TK; ++k) s[k] = 0.f;
+        if (whole) {
+#pragma unroll(TK == 1 ? 8 : 2)
             for (int d = 4 * lane; d < a.D; d += 4 * BN_WAVE) {
-                const float4 wv = *reinterpret_cast<const float4*>(w + d), xv = *reinterpret_cast<const float4*>(hs + d);
-                s = fmaf(xv.x, wv.x, s); s = fmaf(xv.y, wv.y, s); s = fmaf(xv.z, wv.z, s); s = fmaf(xv.w, wv.w, s);
+                const float4 wv = *reinterpret_cast<const float4*>(w + d);
+#pragma unroll
+                for (int k = 0; k < TK; ++k) {
+                    const float4 xv = moe_load4(h[k] + d);
+                    s[k] = fmaf(xv.x, wv.x, s[k]); s[k] = fmaf(xv.y, wv.y, s[k]);
+                    s[k] = fmaf(xv.z, wv.z, s[k]); s[k] = fmaf(xv.w, wv.w, s[k]);
+                }
             }
         } else {
-            for (int d = lane; d < a.D; d += BN_WAVE) s = fmaf(hs[d], w[d], s);
+            for (int d = lane; d < a.D; d += BN_WAVE)
+#pragma unroll
+                for (int k = 0; k < TK; ++k) s[k] = fmaf(to_f32(h[k][d]), w[d], s[k]);
         }
-        s = wave_sum(s);
-        if (lane == 0) {
-            if (e < a.E) zs[e] = a.zbias ? s + a.zbias[e] : s;
-            else a.gate_out[t] = 1.0f / (1.0f + expf(-s));
+#pragma unroll
+        for (int k = 0; k < TK; ++k) {
+            s[k] = wave_sum(s[k]);
+            if (lane == 0) {
+                if (e < a.E) route_smem[k * (a.E + a.groups) + e] = a.zbias ? s[k] + a.zbias[e] : s[k];
+                else if (t0 + k < a.T) a.gate_out[t0 + k] = 1.0f / (1.0f + expf(-s[k]));
+            }
         }
     }
     __syncthreads();
-    if (wave != 0) return;
-    float z[MOE_PER_LANE];                               // expert lane + 64 j
+    const int t = t0 + wave;
+    if (wave >= TK || t >= a.T) return;
+    float* zs = route_smem + wave * (a.E + a.groups);
+    float z[PL];                               // expert lane + 64 j
 #pragma unroll
-    for (int j = 0; j < MOE_PER_LANE; ++j) z[j] = lane + BN_WAVE * j < a.E ? zs[lane + BN_WAVE * j] : -INFINITY;
+    for (int j = 0; j < PL; ++j) z[j] = lane + BN_WAVE * j < a.E ? zs[lane + BN_WAVE * j] : -INFINITY;
     float zmax = -INFINITY, denom = 1.f;
     if (a.scoring == MOE_SCORE_SOFTMAX) {
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j) zmax = fmaxf(zmax, z[j]);
+        for (int j = 0; j < PL; ++j) zmax = fmaxf(zmax, z[j]);
         zmax = wave_max(zmax);
         float sum = 0.f;
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j) sum += z[j] == -INFINITY ? 0.f : expf(z[j] - zmax);
+        for (int j = 0; j < PL; ++j) sum += z[j] == -INFINITY ? 0.f : expf(z[j] - zmax);
         denom = wave_sum(sum);
     }
     // with a choice bias the experts are ranked by score + bias: the scores of all experts are formed first and z holds
     // the ranking value from here on
-    float sc[MOE_PER_LANE];
+    float sc[PL];
     if (a.bias) {
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j) {
+        for (int j = 0; j < PL; ++j) {
             const int e = lane + BN_WAVE * j;
             sc[j] = 0.f;
             if (e < a.E) {
@@ -101,13 +145,13 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
         }
     }
     if (a.groups > 1) {
-        // the ranking values (the logits rank as their scores do) meet in shared memory, where this wave alone is left: a
-        // lane takes groups lane, lane + 64, ..., forms their best members' values, then counts the groups ahead of each
+        // the ranking values (the logits rank as their scores do) meet in the wave's own part of shared memory: a lane
+        // takes groups lane, lane + 64, ..., forms their best members' values, then counts the groups ahead of each
         float* rank = zs;
         float* best = zs + a.E;
         const int size = a.E / a.groups;
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j)
+        for (int j = 0; j < PL; ++j)
             if (lane + BN_WAVE * j < a.E) rank[lane + BN_WAVE * j] = z[j];
         __threadfence_block();
         __builtin_amdgcn_wave_barrier();
@@ -119,7 +163,7 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
         __threadfence_block();
         __builtin_amdgcn_wave_barrier();
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j) {
+        for (int j = 0; j < PL; ++j) {
             const int e = lane + BN_WAVE * j;
             if (e >= a.E) continue;
             const int g = e / size;
@@ -135,7 +179,7 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
         float best = -INFINITY;
         int at = MOE_MAX_EXPERTS;
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j)
+        for (int j = 0; j < PL; ++j)
             if (z[j] > best) { best = z[j]; at = lane + BN_WAVE * j; }
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) {
@@ -146,7 +190,7 @@ __global__ __launch_bounds__(MOE_ROUTE_THREADS) void moe_route_kernel(RouteArgs 
         if (at >= a.E) at = k;                           // a row of NaNs (a padding row's garbage): still an expert that exists
         float own = 0.f;                                 // the chosen expert's plain score, held by the lane that owns it
 #pragma unroll
-        for (int j = 0; j < MOE_PER_LANE; ++j)
+        for (int j = 0; j < PL; ++j)
             if (at == lane + BN_WAVE * j) { z[j] = -INFINITY; if (a.bias) own = sc[j]; }
         const float score = a.bias ? wave_sum(own)
                           : a.scoring == MOE_SCORE_SOFTMAX ? expf(best - zmax) / denom : 1.0f / (1.0f + expf(-best));
@@ -175,15 +219,28 @@ extern "C" int bn_moe_route(int dtype, const void* h, int ld, const float* wr, i
     if (n_tokens <= 0 || D <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || K <= 0 || K > E || ld < D || !h || !wr || !ids || !wts)
         return BN_ERR_ARG;
     if (scoring != MOE_SCORE_SIGMOID && scoring != MOE_SCORE_SOFTMAX) return BN_ERR_ARG;
-    if ((size_t)(D + 4 + E + groups) * sizeof(float) > 64 * 1024 || ((uintptr_t)wr & 15)) return BN_ERR_ARG;
+    if ((uintptr_t)wr & 15) return BN_ERR_ARG;
     RouteArgs a;
-    a.h = h; a.wr = wr; a.ids = ids; a.wts = wts; a.ld = ld; a.D = D; a.E = E; a.K = K; a.scoring = scoring; a.renorm = renorm ? 1 : 0;
+    a.h = h; a.wr = wr; a.ids = ids; a.wts = wts; a.ld = ld; a.T = n_tokens; a.D = D; a.E = E; a.K = K; a.scoring = scoring; a.renorm = renorm ? 1 : 0;
     a.bias = bias; a.zbias = zbias; a.gate_w = gate_w; a.gate_out = gate_out; a.floor = floor; a.scale = scale;
     a.groups = groups; a.keep = keep;
-    const size_t shm = (size_t)(((D + 3) & ~3) + E + groups) * sizeof(float);
-    if (dtype == BN_DT_F32) hipLaunchKernelGGL(moe_route_kernel<float>, dim3(n_tokens), dim3(MOE_ROUTE_THREADS), shm, s, a);
-    else if (dtype == BN_DT_BF16) hipLaunchKernelGGL(moe_route_kernel<bf16>, dim3(n_tokens), dim3(MOE_ROUTE_THREADS), shm, s, a);
-    else return BN_ERR_DTYPE;
+    if (dtype != BN_DT_F32 && dtype != BN_DT_BF16) return BN_ERR_DTYPE;
+    const size_t rows = (size_t)MOE_ROUTE_TOKENS * moe_route_row_bytes(D, dtype == BN_DT_F32 ? 4 : 2);
+    const bool few = n_tokens <= MOE_ROUTE_FEW_ROWS || rows + (size_t)MOE_ROUTE_TOKENS * (E + groups) * sizeof(float) > 64 * 1024;
+    const int tk = few ? 1 : MOE_ROUTE_TOKENS;
+    const size_t shm = (few ? 0 : rows) + (size_t)tk * (E + groups) * sizeof(float);
+    const dim3 grid((n_tokens + tk - 1) / tk), block(E > 4 ? MOE_ROUTE_THREADS : 4 * BN_WAVE);
+#define MOE_ROUTE_GO(PL_)                                                                                                   \
+    do {                                                                                                                    \
+        if (few && dtype == BN_DT_F32) hipLaunchKernelGGL((moe_route_kernel<float, PL_, 1>), grid, block, shm, s, a);       \
+        else if (few) hipLaunchKernelGGL((moe_route_kernel<bf16, PL_, 1>), grid, block, shm, s, a);                         \
+        else if (dtype == BN_DT_F32) hipLaunchKernelGGL((moe_route_kernel<float, PL_, MOE_ROUTE_TOKENS>), grid, block, shm, s, a); \
+        else hipLaunchKernelGGL((moe_route_kernel<bf16, PL_, MOE_ROUTE_TOKENS>), grid, block, shm, s, a);                   \
+    } while (0)
+    if (E <= BN_WAVE) MOE_ROUTE_GO(1);
+    else if (E <= 4 * BN_WAVE) MOE_ROUTE_GO(4);
+    else MOE_ROUTE_GO(MOE_MAX_EXPERTS / BN_WAVE);
+#undef MOE_ROUTE_GO
     return bn_launch_status();
 }
 
@@ -465,11 +522,38 @@ __global__ void gated_unit_kernel(T* __restrict__ out, const T* __restrict__ gu,
     out[i] = from_f32<T>(v);
 }
 
+// the same for bf16 rows of whole 16-byte groups: a thread takes eight consecutive columns
+__global__ __launch_bounds__(256) void gated_unit_bf16x8_kernel(bf16* __restrict__ out, const bf16* __restrict__ gu, int ld,
+                                                                const float* __restrict__ row_scale, int F, float limit, float slope,
+                                                                float shift) {
+    const int r = blockIdx.y, f = 8 * (blockIdx.x * 256 + threadIdx.x);
+    if (f >= F) return;
+    const bf16* row = gu + (size_t)r * ld;
+    const uint4 g = *reinterpret_cast<const uint4*>(row + f), u = *reinterpret_cast<const uint4*>(row + F + f);
+    const uint32_t gw[4] = {g.x, g.y, g.z, g.w}, uw[4] = {u.x, u.y, u.z, u.w};
+    const float s = row_scale ? row_scale[r] : 1.0f;
+    bf16 o[8];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        float a = moe_clamped_unit(bf16lo_to_f32(gw[k]), bf16lo_to_f32(uw[k]), limit, slope, shift);
+        float b = moe_clamped_unit(bf16hi_to_f32(gw[k]), bf16hi_to_f32(uw[k]), limit, slope, shift);
+        if (row_scale) { a *= s; b *= s; }
+        o[2 * k] = from_f32<bf16>(a);
+        o[2 * k + 1] = from_f32<bf16>(b);
+    }
+    *reinterpret_cast<uint4*>(out + (size_t)r * F + f) = *reinterpret_cast<const uint4*>(o);
+}
+
 extern "C" int bn_gated_unit(int dtype, void* out, const void* gu, int ld, const float* row_scale, int n_rows, int F, float limit,
                              float slope, float shift, hipStream_t s) {
     if (n_rows <= 0 || F <= 0 || ld < 2 * F || !out || !gu || !(limit > 0.f)) return BN_ERR_ARG;
     const size_t n = (size_t)n_rows * F;
     const dim3 grid((unsigned)((n + 255) / 256)), block(256);
+    if (dtype == BN_DT_BF16 && F % 8 == 0 && ld % 8 == 0 && n_rows <= 65535 && !(((uintptr_t)out | (uintptr_t)gu) & 15)) {
+        hipLaunchKernelGGL(gated_unit_bf16x8_kernel, dim3((F + 2047) / 2048, n_rows), block, 0, s, (bf16*)out, (const bf16*)gu, ld,
+                           row_scale, F, limit, slope, shift);
+        return bn_launch_status();
+    }
     if (dtype == BN_DT_F32)
         hipLaunchKernelGGL(gated_unit_kernel<float>, grid, block, 0, s, (float*)out, (const float*)gu, ld, row_scale, n_rows, F, limit, slope, shift);
     else if (dtype == BN_DT_BF16)

@@ -3,8 +3,7 @@
 Whole sequences, no cache, nothing carried between calls, one function per mechanism, CPU tensors in float64.  It shares
 no code with the package under test: its own reading of config.json, its own safetensors reading (through the
 `safetensors` library), its own greedy loop.  Notation: h is a sublayer's input [T, D]; positions count from 0; linear
-weights are [out, in]; the recurrence is written token by token and attention query by query, the way their definitions
-read.
+weights are [out, in]; the recurrence is written token by token, the way its definition reads.
 """
 from __future__ import annotations
 
@@ -76,10 +75,12 @@ def rotate_neighbours(x, positions, rot: dict, angle_dtype=F64):
 # ---- mixers ----------------------------------------------------------------------------------------------------
 
 def sink_weights(s, sink):
-    """Softmax weights of scores s [n] whose denominator also holds exp(sink)."""
-    top = torch.maximum(s.max(), sink)
+    """Causal softmax weights of scores s [T, T] (query, key) whose denominators also hold exp(sink)."""
+    T = s.shape[0]
+    s = s.masked_fill(torch.arange(T)[None, :] > torch.arange(T)[:, None], -float("inf"))
+    top = torch.maximum(s.max(dim=1).values, sink)[:, None]
     e = torch.exp(s - top)
-    return e / (e.sum() + torch.exp(sink - top))
+    return e / (e.sum(dim=1, keepdim=True) + torch.exp(sink - top))
 
 
 def latent_attention(h, W, p, m, eps, angle_dtype=F64):
@@ -101,10 +102,9 @@ def latent_attention(h, W, p, m, eps, angle_dtype=F64):
     k = (c @ W[p + "uk"].T).reshape(T, H, d)
     v = (c @ W[p + "uv"].T).reshape(T, H, vd)
     out = torch.zeros((T, H, vd), dtype=F64)
-    for t in range(T):
-        for i in range(H):
-            s = (k[:t + 1, i] @ q[t, i, :d] + k_rot[:t + 1, 0] @ q_rot[t, i]) * m["scale"]
-            out[t, i] = sink_weights(s, W[p + "sink"][i]) @ v[:t + 1, i]
+    for i in range(H):
+        s = (q[:, i, :d] @ k[:, i].T + q_rot[:, i] @ k_rot[:, 0].T) * m["scale"]
+        out[:, i] = sink_weights(s, W[p + "sink"][i]) @ v[:, i]
     return out.reshape(T, H * vd) @ W[p + "o"].T
 
 

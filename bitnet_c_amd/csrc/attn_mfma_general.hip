@@ -395,31 +395,36 @@ __global__ __launch_bounds__(BN_WAVE) void attn_general_decode_kernel(GenDecodeA
 }
 
 // out[row, d] = sum_s e^(m_s - m) o_s[d] / (sum_s e^(m_s - m) l_s [+ e^(-m) for the sink]) [sigmoid(gate)], the splits in index order;
-// one wave a (token, head) row, a lane four value columns at a time
+// one wave a (token, head) row: the splits' factors are formed a lane a split, then a lane takes four value columns at a time
+// with several splits' loads in flight (a split without keys holds zeros, and its factor is 0)
+#define AG_MAX_SPLITS BN_WAVE
 __global__ __launch_bounds__(BN_WAVE) void attn_general_combine_kernel(bf16* __restrict__ out, int out_stride,
                                                                        const float* __restrict__ part_o,
                                                                        const float* __restrict__ part_ml, int H, int vd,
                                                                        int n_splits, int sink,
                                                                        const float* __restrict__ sink_values,
                                                                        const bf16* __restrict__ gate, int gate_stride) {
-    const int row = blockIdx.x, tok = row / H, head = row - tok * H;
+    __shared__ float factor[AG_MAX_SPLITS], share[AG_MAX_SPLITS];
+    const int row = blockIdx.x, tok = row / H, head = row - tok * H, lane = threadIdx.x;
     const float* ml = part_ml + (size_t)row * n_splits * 2;
     const float sv = sink && sink_values ? sink_values[head] : 0.f;
-    float m = sink ? sv : -INFINITY;
-    for (int s = 0; s < n_splits; ++s) m = fmaxf(m, ml[2 * s]);
+    const float mine = lane < n_splits ? ml[2 * lane] : -INFINITY, sum = lane < n_splits ? ml[2 * lane + 1] : 0.f;
+    const float m = wave_max(sink ? fmaxf(sv, mine) : mine);
+    const float f = m != -INFINITY ? expf(mine - m) : 0.f;
+    factor[lane] = f;
+    share[lane] = f * sum;
+    __syncthreads();
     float den = sink ? expf(sv - m) : 0.f;
-    if (m != -INFINITY)
-        for (int s = 0; s < n_splits; ++s) den = fmaf(expf(ml[2 * s] - m), ml[2 * s + 1], den);
+    for (int s = 0; s < n_splits; ++s) den += share[s];
     const float inv = den > 0.f ? 1.0f / den : 0.f;
-    for (int d = 4 * threadIdx.x; d < vd; d += 4 * BN_WAVE) {
+    for (int d = 4 * lane; d < vd; d += 4 * BN_WAVE) {
         float4 num = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (m != -INFINITY) {
-            for (int s = 0; s < n_splits; ++s) {
-                const float w = expf(ml[2 * s] - m);      // 0 for a split without keys
-                if (w == 0.f) continue;
-                const float4 o = *reinterpret_cast<const float4*>(part_o + ((size_t)row * n_splits + s) * vd + d);
-                num.x = fmaf(w, o.x, num.x); num.y = fmaf(w, o.y, num.y); num.z = fmaf(w, o.z, num.z); num.w = fmaf(w, o.w, num.w);
-            }
+        const float* op0 = part_o + (size_t)row * n_splits * vd + d;
+#pragma unroll 8
+        for (int s = 0; s < n_splits; ++s) {
+            const float4 o = *reinterpret_cast<const float4*>(op0 + (size_t)s * vd);
+            const float w = factor[s];
+            num.x = fmaf(w, o.x, num.x); num.y = fmaf(w, o.y, num.y); num.z = fmaf(w, o.z, num.z); num.w = fmaf(w, o.w, num.w);
         }
         bf16* op = out + (size_t)tok * out_stride + (size_t)head * vd + d;
         ag_store4(op, gate ? gate + (size_t)tok * gate_stride + (size_t)head * vd + d : nullptr, num.x * inv, num.y * inv, num.z * inv,
@@ -509,7 +514,7 @@ extern "C" int bn_attn_general_decode(const void* q, int q_stride, void* out, in
         return BN_ERR_ARG;
     if (n_splits > 1 && (!part_o || !part_ml || ((uintptr_t)part_o & 15) || (!max_len && (chunk <= 0 || chunk % BN_PAGE)))) return BN_ERR_ARG;
     const int head_tiles = (H / Hkv + 15) / 16;
-    if ((long long)Hkv * head_tiles > 65535 || n_splits > 65535) return BN_ERR_ARG;
+    if ((long long)Hkv * head_tiles > 65535 || n_splits > AG_MAX_SPLITS) return BN_ERR_ARG;
     if (gate && (gate_stride % 4 || ((uintptr_t)gate & 7))) return BN_ERR_ARG;
     GenDecodeArgs a;
     a.gate = (const bf16*)gate; a.gate_stride = gate_stride; a.keep_first = keep_first;

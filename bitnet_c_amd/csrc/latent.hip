@@ -121,7 +121,7 @@ struct HeadLinearArgs {
     const void* gate;         // [T, ldg]: the gate of output column n is entry n / gate_group (1: one a column; O: one a head); null: none
     int ldx, ldy, ldg, T, H, I, O, gate_group;
     Rotation r;               // rot > 0: columns rot_off .. rot_off + rot of every head's output turn by the row's position
-    int rot_off;
+    int rot_off, OC;          // OC: output columns of a workgroup of the wide kernel
     const int* positions;     // [T]; < 0: a padding row, whose columns stay as they are
 };
 
@@ -173,8 +173,8 @@ __global__ __launch_bounds__(HL_COLS * HL_SLICES) void head_linear_kernel(HeadLi
 
 // The same product with 16-byte loads of the weights: a lane owns HLW_VEC consecutive output columns (8 bf16 or 4 float32),
 // O / HLW_VEC lanes cover a row of the head's matrix, and the 256 / (O / HLW_VEC) groups of lanes take the input dimension
-// in turn; their sums meet in shared memory.  One workgroup a (head, four rows of x): at one row a head's matrix is read
-// with sixteen loads a lane instead of one load an input row.
+// in turn; their sums meet in shared memory.  One workgroup a (head, four rows of x, run of OC output columns): at few rows
+// the columns are cut into runs until the launch has workgroups enough for the chip.
 #define HLW_ROWS 4
 #define HLW_THREADS 256
 
@@ -198,10 +198,10 @@ template <> struct HlwVec<float> {
 template <typename T>
 __global__ __launch_bounds__(HLW_THREADS) void head_linear_wide_kernel(HeadLinearArgs a) {
     constexpr int V = HlwVec<T>::N;
-    extern __shared__ float xs[];                        // [HLW_ROWS][I], then the groups' sums [groups][HLW_ROWS][O]
+    extern __shared__ float xs[];                        // [HLW_ROWS][I], then the groups' sums [groups][HLW_ROWS][OC]
     float* red = xs + HLW_ROWS * a.I;
-    const int h = blockIdx.x, t0 = blockIdx.y * HLW_ROWS;
-    const int lanes = a.O / V, groups = HLW_THREADS / lanes;         // lanes <= 256
+    const int h = blockIdx.x, t0 = blockIdx.y * HLW_ROWS, o0 = blockIdx.z * a.OC, OC = min(a.OC, a.O - o0);
+    const int lanes = OC / V, groups = HLW_THREADS / lanes;          // lanes <= 256
     const int grp = threadIdx.x / lanes, cg = threadIdx.x - grp * lanes;
     const int rows = min(HLW_ROWS, a.T - t0);
     const T* x = reinterpret_cast<const T*>(a.x);
@@ -216,7 +216,7 @@ __global__ __launch_bounds__(HLW_THREADS) void head_linear_wide_kernel(HeadLinea
 #pragma unroll
         for (int k = 0; k < V; ++k) acc[r][k] = 0.f;
     if (grp < groups) {
-        const T* w = reinterpret_cast<const T*>(a.w) + (size_t)h * a.I * a.O + (size_t)cg * V;
+        const T* w = reinterpret_cast<const T*>(a.w) + (size_t)h * a.I * a.O + o0 + (size_t)cg * V;
 #pragma unroll 4
         for (int i = grp; i < a.I; i += groups) {
             float wv[V];
@@ -231,23 +231,23 @@ __global__ __launch_bounds__(HLW_THREADS) void head_linear_wide_kernel(HeadLinea
 #pragma unroll
         for (int r = 0; r < HLW_ROWS; ++r)
 #pragma unroll
-            for (int k = 0; k < V; ++k) red[((size_t)grp * HLW_ROWS + r) * a.O + cg * V + k] = acc[r][k];
+            for (int k = 0; k < V; ++k) red[((size_t)grp * HLW_ROWS + r) * OC + cg * V + k] = acc[r][k];
     }
     __syncthreads();
     T* y = reinterpret_cast<T*>(a.y);
     const T* g = reinterpret_cast<const T*>(a.gate);
-    for (int idx = threadIdx.x; idx < rows * a.O; idx += HLW_THREADS) {
-        const int r = idx / a.O, o = idx - r * a.O;
+    for (int idx = threadIdx.x; idx < rows * OC; idx += HLW_THREADS) {
+        const int r = idx / OC, c = idx - r * OC, o = o0 + c;
         float v = 0.f;
-        for (int k = 0; k < groups; ++k) v += red[((size_t)k * HLW_ROWS + r) * a.O + o];
+        for (int k = 0; k < groups; ++k) v += red[((size_t)k * HLW_ROWS + r) * OC + c];
         if (g) v *= 1.0f / (1.0f + expf(-to_f32(g[(size_t)(t0 + r) * a.ldg + ((size_t)h * a.O + o) / a.gate_group])));
         const int ro = o - a.rot_off, pos = ro >= 0 && ro < a.r.rot ? a.positions[t0 + r] : -1;
-        if (pos >= 0) {                                  // this column and its partner, both from the sums
+        if (pos >= 0) {                                  // this column and its partner, both from this workgroup's sums
             const int i = a.r.interleaved ? ro >> 1 : ro < a.r.rot / 2 ? ro : ro - a.r.rot / 2;
             const bool second = ro != rot_first(a.r, i);
-            const int po = a.rot_off + (second ? rot_first(a.r, i) : rot_second(a.r, i));
+            const int pc = a.rot_off + (second ? rot_first(a.r, i) : rot_second(a.r, i)) - o0;
             float p = 0.f;
-            for (int k = 0; k < groups; ++k) p += red[((size_t)k * HLW_ROWS + r) * a.O + po];
+            for (int k = 0; k < groups; ++k) p += red[((size_t)k * HLW_ROWS + r) * OC + pc];
             float u = second ? p : v, w = second ? v : p;
             rot_turn(a.r, i, pos, u, w);
             v = second ? w : u;
@@ -256,12 +256,27 @@ __global__ __launch_bounds__(HLW_THREADS) void head_linear_wide_kernel(HeadLinea
     }
 }
 
+// The columns of a workgroup: all of them, or halves of that (down to 32, which leaves a row of the matrix 64 bytes a
+// workgroup) while the launch would have fewer than HLW_WORKGROUPS; a run holds both columns of every rotated pair.
+#define HLW_WORKGROUPS 256
+static int hlw_columns(const HeadLinearArgs& a, int row_tiles) {
+    int oc = a.O;
+    while (oc % 64 == 0 && (long long)a.H * row_tiles * ((a.O + oc - 1) / oc) < HLW_WORKGROUPS) {
+        const int half = oc / 2;
+        const bool whole_pairs = a.r.rot == 0 || (a.r.interleaved && a.rot_off % 2 == 0) ||
+                                 a.rot_off / half == (a.rot_off + a.r.rot - 1) / half;
+        if (!whole_pairs) break;
+        oc = half;
+    }
+    return oc;
+}
+
 template <typename T>
-static bool hlw_takes(const void* w, int I, int O) {
+static bool hlw_takes(const void* w, int I, int O, int OC) {
     constexpr int V = HlwVec<T>::N;
-    if (O % V || O / V > HLW_THREADS || ((uintptr_t)w & 15)) return false;
-    const int groups = HLW_THREADS / (O / V);
-    return (size_t)HLW_ROWS * ((size_t)I + (size_t)groups * O) * sizeof(float) <= 64 * 1024;
+    if (O % V || OC % V || OC / V > HLW_THREADS || ((uintptr_t)w & 15)) return false;
+    const int groups = HLW_THREADS / (OC / V);
+    return (size_t)HLW_ROWS * ((size_t)I + (size_t)groups * OC) * sizeof(float) <= 64 * 1024;
 }
 
 extern "C" int bn_rope_heads(int dtype, void* x, int ld, const int* positions, const float* inv_freq, int n_rows, int H,
@@ -281,11 +296,13 @@ extern "C" int bn_head_linear(int dtype, const void* x, int ldx, const void* w, 
     a.r.rot = rot; a.r.inv_freq = inv_freq; a.r.mult = rot_mult; a.r.interleaved = interleaved ? 1 : 0; a.rot_off = rot_off;
     a.positions = positions;
     if (dtype != BN_DT_F32 && dtype != BN_DT_BF16) return BN_ERR_DTYPE;
-    const bool wide = dtype == BN_DT_F32 ? hlw_takes<float>(w, I, O) : hlw_takes<bf16>(w, I, O);
-    if (wide && (n_rows + HLW_ROWS - 1) / HLW_ROWS <= 65535) {
-        const int vec = dtype == BN_DT_F32 ? 4 : 8, groups = HLW_THREADS / (O / vec);
-        const dim3 wgrid(H, (n_rows + HLW_ROWS - 1) / HLW_ROWS);
-        const size_t wshm = (size_t)HLW_ROWS * ((size_t)I + (size_t)groups * O) * sizeof(float);
+    const int wide_tiles = (n_rows + HLW_ROWS - 1) / HLW_ROWS;
+    a.OC = hlw_columns(a, wide_tiles);
+    const bool wide = dtype == BN_DT_F32 ? hlw_takes<float>(w, I, O, a.OC) : hlw_takes<bf16>(w, I, O, a.OC);
+    if (wide && wide_tiles <= 65535) {
+        const int vec = dtype == BN_DT_F32 ? 4 : 8, groups = HLW_THREADS / (a.OC / vec);
+        const dim3 wgrid(H, wide_tiles, O / a.OC);
+        const size_t wshm = (size_t)HLW_ROWS * ((size_t)I + (size_t)groups * a.OC) * sizeof(float);
         if (dtype == BN_DT_F32) hipLaunchKernelGGL(head_linear_wide_kernel<float>, wgrid, dim3(HLW_THREADS), wshm, s, a);
         else hipLaunchKernelGGL(head_linear_wide_kernel<bf16>, wgrid, dim3(HLW_THREADS), wshm, s, a);
         return bn_launch_status();

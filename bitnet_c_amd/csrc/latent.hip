@@ -257,11 +257,13 @@ __global__ __launch_bounds__(HLW_THREADS) void head_linear_wide_kernel(HeadLinea
 }
 
 // The columns of a workgroup: all of them, or halves of that (down to 32, which leaves a row of the matrix 64 bytes a
-// workgroup) while the launch would have fewer than HLW_WORKGROUPS; a run holds both columns of every rotated pair.
+// workgroup) while the launch would have fewer than HLW_WORKGROUPS; a run holds both columns of every rotated pair.  The cut
+// decides how many groups of lanes share a column's sum: float32 rows are not cut, so that their sums keep one order whatever
+// number of rows a step has.
 #define HLW_WORKGROUPS 256
-static int hlw_columns(const HeadLinearArgs& a, int row_tiles) {
+static int hlw_columns(const HeadLinearArgs& a, int dtype, int row_tiles) {
     int oc = a.O;
-    while (oc % 64 == 0 && (long long)a.H * row_tiles * ((a.O + oc - 1) / oc) < HLW_WORKGROUPS) {
+    while (dtype == BN_DT_BF16 && oc % 64 == 0 && (long long)a.H * row_tiles * ((a.O + oc - 1) / oc) < HLW_WORKGROUPS) {
         const int half = oc / 2;
         const bool whole_pairs = a.r.rot == 0 || (a.r.interleaved && a.rot_off % 2 == 0) ||
                                  a.rot_off / half == (a.rot_off + a.r.rot - 1) / half;
@@ -297,7 +299,7 @@ extern "C" int bn_head_linear(int dtype, const void* x, int ldx, const void* w, 
     a.positions = positions;
     if (dtype != BN_DT_F32 && dtype != BN_DT_BF16) return BN_ERR_DTYPE;
     const int wide_tiles = (n_rows + HLW_ROWS - 1) / HLW_ROWS;
-    a.OC = hlw_columns(a, wide_tiles);
+    a.OC = hlw_columns(a, dtype, wide_tiles);
     const bool wide = dtype == BN_DT_F32 ? hlw_takes<float>(w, I, O, a.OC) : hlw_takes<bf16>(w, I, O, a.OC);
     if (wide && wide_tiles <= 65535) {
         const int vec = dtype == BN_DT_F32 ? 4 : 8, groups = HLW_THREADS / (a.OC / vec);

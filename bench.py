@@ -296,7 +296,7 @@ def _zenasun_configs(z):
     layers = [dict(type="latent_attention", mixer=lat, mlp=moe) if i % 3 == 2 else dict(type="retention", mixer=ret, mlp=moe)
               for i in range(z["layers"])]
     zen = dict(architecture="Zenasun", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6), embedding=dict(scale=8.0),
-               logit_softcap=30.0, layers=layers)
+               logit_softcap=50.0, layers=layers)
     mut, faz, _, llama = _mutirax_configs(z)
     return zen, mut, faz, llama
 

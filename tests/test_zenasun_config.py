@@ -132,7 +132,7 @@ def test_stored_rows_of_a_latent():
     the rest are the vector kernel's as they are."""
     from bitnet_c_amd import ops
     assert ops.latent_row_widths(192, 64) == (256, 192) and ops.latent_row_widths(96, 32) == (128, 96)
-    assert ops.latent_row_widths(128, 16) == (160, 128) and ops.latent_row_widths(160, 32) == (192, 192)
+    assert ops.latent_row_widths(120, 24) == (160, 128) and ops.latent_row_widths(160, 32) == (192, 192)
     assert ops.latent_row_widths(80, 16) == (96, 96) and ops.latent_row_widths(14, 2) == (16, 14)
     assert ops.latent_row_widths(512, 64) == (576, 512) and ops.latent_row_widths(40, 8) == (48, 40)
     for rank in range(2, 513, 2):

@@ -65,7 +65,7 @@ CONFIGS = {
         _ret(2, 64, 64, (10000.0, 64), _moe(12, 4, 3, 64, 4, 2)),
         _lat(4, 32, 32, 32, 96, 48, 0.12, 100000.0, _moe(6, 2, 2, 64, 2, 1)),
         _ret(1, 128, 128, (10000.0, 96), None),
-        _lat(3, 64, 16, 64, 128, 64, 0.11, 1000000.0, _moe(28, 4, 4, 32, 8, 3)),
+        _lat(3, 64, 24, 64, 120, 64, 0.11, 200000.0, _moe(28, 4, 4, 32, 8, 3)),
         _ret(2, 64, 64, (10000.0, 64), _moe(12, 4, 3, 64, 4, 2), weights_of=0)]),
     # ones everywhere: one head, one expert beside one identity expert, a decay of exactly 1 (nothing fades) and 0
     # (nothing is kept), the first layer runs the last one's weights
